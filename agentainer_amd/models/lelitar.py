@@ -54,6 +54,8 @@ from .llama import AttnMetadata
 
 # the MFMA tile kernel contracts the latent rank in chunks of 32
 RANK_ALIGN = 32
+CAUSAL_WINDOW = 1 << 30  # a window no sequence outgrows
+ROW_ALIGN = 8            # rows of a stacked projection: 16-byte aligned bf16
 
 
 @dataclass
@@ -65,6 +67,8 @@ class LatentMixerConfig:
     kv_rank: int      # cached key/value latent size
     window: int       # a query at p sees keys p-window < j <= p
     scale: float
+    gate: str = "elem"   # output gate per "elem"ent or per "head"
+    sink: bool = False   # a learned score per head in the denominator
 
     @property
     def padded_rank(self) -> int:
@@ -156,14 +160,22 @@ def config_from_checkpoint(path: str) -> LelitarConfig:
 
 
 class LatentAttention(torch.nn.Module):
-    """Sliding-window latent attention with a sigmoid output gate."""
+    """Sliding-window latent attention with a sigmoid output gate (per
+    output element, or one per head) and, optionally, a softmax sink. The
+    head gate and the sink are applied by the attention kernels where they
+    normalize the weighted sum: both are numbers per (token, head), so they
+    commute with the value up-projection."""
 
     def __init__(self, width: int, mc: LatentMixerConfig, eps: float, dtype):
         super().__init__()
         self.mc = mc
         self.eps = eps
         H, Rp = mc.heads, mc.padded_rank
-        self.n_in = mc.q_rank + mc.kv_rank + H * mc.vdim
+        n_gate = H if mc.gate == "head" else H * mc.vdim
+        self.g_off = mc.q_rank + mc.kv_rank
+        self.n_gate = n_gate
+        n = self.g_off + n_gate
+        self.n_in = -(-n // ROW_ALIGN) * ROW_ALIGN if mc.gate == "head" else n
 
         def P(*shape, dt=dtype):
             return torch.nn.Parameter(torch.empty(*shape, dtype=dt),
@@ -178,12 +190,17 @@ class LatentAttention(torch.nn.Module):
         self.w_uk = P(H, mc.dim, Rp)     # q_lat[h] = q[h] @ w_uk[h]
         self.w_uv = P(H, Rp, mc.vdim)    # a[h] = o_lat[h] @ w_uv[h]
         self.w_o = P(width, H * mc.vdim)
+        self.sink = P(H, dt=torch.float32) if mc.sink else None
 
     @torch.no_grad()
     def load(self, get):
         mc = self.mc
         H, R, Rp = mc.heads, mc.kv_rank, mc.padded_rank
-        self.w_in.copy_(torch.cat([get("dq"), get("dkv"), get("g")], dim=0))
+        self.w_in.zero_()
+        self.w_in[:self.g_off + self.n_gate].copy_(
+            torch.cat([get("dq"), get("dkv"), get("g")], dim=0))
+        if self.sink is not None:
+            self.sink.copy_(get("sink").float())
         self.q_norm.copy_(get("dq.norm").float())
         self.kv_norm.copy_(get("dkv.norm").float())
         self.w_uq.copy_(get("uq"))
@@ -205,14 +222,22 @@ class LatentAttention(torch.nn.Module):
         q = ops.linear(cq, self.w_uq).view(T, H, mc.dim)
         q_lat = torch.bmm(q.transpose(0, 1), self.w_uk)        # [H, T, Rp]
         o_lat = torch.empty_like(q_lat)
+        gate = proj[:, self.g_off:self.g_off + self.n_gate]
+        by_head = mc.gate == "head"
         ops.latent_window_attention(
             o_lat, q_lat, cache, md.page_table, md.seq_lens,
             md.query_starts if md.is_prefill else None,
             md.query_lens if md.is_prefill else None,
-            mc.scale, mc.window, max_qlen=md.max_qlen if md.is_prefill else 1)
+            mc.scale, mc.window, max_qlen=md.max_qlen if md.is_prefill else 1,
+            sink=self.sink, head_gate=gate if by_head else None)
+        if by_head:
+            # the products land token-major: ready for the output projection
+            a = torch.empty(T, H, mc.vdim, dtype=h.dtype, device=h.device)
+            torch.bmm(o_lat, self.w_uv, out=a.transpose(0, 1))
+            return ops.linear(a.view(T, H * mc.vdim), self.w_o)
         a = torch.bmm(o_lat, self.w_uv)                        # [H, T, vdim]
         gated = torch.empty(T, H * mc.vdim, dtype=h.dtype, device=h.device)
-        ops.sigmoid_gate_mul(gated, a, proj[:, mc.q_rank + mc.kv_rank:])
+        ops.sigmoid_gate_mul(gated, a, gate)
         return ops.linear(gated, self.w_o)
 
 

@@ -81,7 +81,7 @@ DEFAULT_RANK = 16       # low-rank stages of named random-init configs
 
 @dataclass
 class MatrixMemoryConfig:
-    kind: int                 # ops.SCAN_GLA / SCAN_DELTA / SCAN_MLSTM
+    kind: int                 # ops.SCAN_GLA / _DELTA / _DELTA_HEAD / _MLSTM
     heads: int                # value heads (= memories per layer)
     qk_heads: int             # query/key heads; heads % qk_heads == 0
     dim: int                  # key channels per head
@@ -296,7 +296,10 @@ def _step_shape(md: AttnMetadata):
 
 class MatrixMemoryMixer(torch.nn.Module):
     """Linear-recurrent mixer over a per-head matrix memory S [dim, vdim]
-    (see MatrixMemoryConfig.kind); the memory is per-sequence state."""
+    (see MatrixMemoryConfig.kind); the memory is per-sequence state.
+    SCAN_DELTA_HEAD is the delta rule with one decay per head: its decay and
+    write-strength projections are the narrow GEMM's 2H rows, its output
+    gate a full-rank SiLU gate that rides in the wide GEMM."""
 
     def __init__(self, width: int, mc: MatrixMemoryConfig, eps: float, dtype):
         super().__init__()
@@ -308,28 +311,34 @@ class MatrixMemoryMixer(torch.nn.Module):
         kind = mc.kind
         # wide projections, one GEMM in the compute dtype: q | k | v
         # (| full-rank output gate)
-        self.full_gate = kind in (ops.SCAN_GLA, ops.SCAN_MLSTM)
+        self.full_gate = kind != ops.SCAN_DELTA
         n = self.q_sz + self.k_sz + self.v_sz + (self.v_sz if self.full_gate
                                                  else 0)
         self.w_in = _param(_pad(n), width, dtype=dtype)
-        # narrow projections that feed decays and gates, one fp32 GEMM on
-        # the fp32 residual
+        # narrow projections that feed decays and gates, one GEMM with an
+        # fp32 result: on the fp32 residual, or on the mixer input (one
+        # decay per head)
         if kind == ops.SCAN_GLA:
             n_small = mc.decay_rank
         elif kind == ops.SCAN_DELTA:
             n_small = mc.decay_rank + mc.gate_rank + H
         else:
             n_small = 2 * H
-        self.w_small = _param(n_small, width, dtype=f32)
+        self.w_small = _param(n_small, width, dtype=(
+            dtype if kind == ops.SCAN_DELTA_HEAD else f32))
         if kind == ops.SCAN_MLSTM:
             self.gate_bias = _param(2 * H, dtype=f32)
             self.norm_w = _param(H * Dv, dtype=f32)
+        elif kind == ops.SCAN_DELTA_HEAD:
+            self.gate_bias = _param(H, dtype=f32)
+            self.norm_w = _param(Dv, dtype=f32)
         else:
             self.a2 = _param(H * D, mc.decay_rank, dtype=f32)
             self.gate_bias = _param(H * D, dtype=f32)
             self.norm_w = _param(Dv, dtype=f32)
         if kind == ops.SCAN_DELTA:
             self.g2 = _param(H * Dv, mc.gate_rank, dtype=f32)
+        if kind in (ops.SCAN_DELTA, ops.SCAN_DELTA_HEAD):
             self.head_rate = _param(H, dtype=f32)
         self.conv_channels = self.q_sz + self.k_sz + self.v_sz
         self.w_conv = (_param(mc.conv_taps, self.conv_channels, dtype=f32)
@@ -358,6 +367,10 @@ class MatrixMemoryMixer(torch.nn.Module):
             self.g2.copy_(f("g2"))
             self.gate_bias.copy_(f("dt_bias"))
             self.head_rate.copy_(f("A_log"))
+        elif mc.kind == ops.SCAN_DELTA_HEAD:
+            self.w_small.copy_(torch.cat([f("a"), f("b")], dim=0))
+            self.gate_bias.copy_(f("dt_bias"))
+            self.head_rate.copy_(f("A_log"))
         else:
             self.w_small.copy_(torch.cat([f("i"), f("f")], dim=0))
             self.gate_bias.copy_(torch.cat([f("i.b"), f("f.b")], dim=0))
@@ -368,16 +381,18 @@ class MatrixMemoryMixer(torch.nn.Module):
                                          f("v.conv")], dim=0).t())
         self.w_o.copy_(get("o"))
 
-    def forward(self, h: torch.Tensor, x: torch.Tensor, state: dict,
-                md: AttnMetadata) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, x: Optional[torch.Tensor],
+                state: dict, md: AttnMetadata) -> torch.Tensor:
         """h: the mixer input in the compute dtype; x: the same rows of the
-        fp32 residual; state: this layer's per-sequence state tensors."""
+        fp32 residual (not read by SCAN_DELTA_HEAD); state: this layer's per-sequence state tensors."""
         mc = self.mc
         T, H, G, D, Dv = h.size(0), mc.heads, mc.qk_heads, mc.dim, mc.vdim
         kind = mc.kind
         q_starts, q_lens = _step_shape(md)
         proj = ops.linear(h, self.w_in)
-        small = F.linear(x, self.w_small)
+        small = (ops.narrow_linear(h, self.w_small)
+                 if kind == ops.SCAN_DELTA_HEAD
+                 else F.linear(x, self.w_small))
         k0, v0 = self.q_sz, self.q_sz + self.k_sz
         g0 = v0 + self.v_sz
         qkv, q_scale = proj, D ** -0.5
@@ -404,6 +419,10 @@ class MatrixMemoryMixer(torch.nn.Module):
             out_gate = F.linear(small[:, r:r + rg], self.g2)
             beta = small[:, r + rg:]
             head_rate, param = self.head_rate, 0.0
+        elif kind == ops.SCAN_DELTA_HEAD:
+            gate, beta = small[:, :H], small[:, H:]
+            head_rate, param = self.head_rate, 0.0
+            out_gate = proj[:, g0:g0 + self.v_sz]
         else:
             gate, param = small, mc.gate_cap
             out_gate = proj[:, g0:g0 + self.v_sz]
@@ -415,7 +434,8 @@ class MatrixMemoryMixer(torch.nn.Module):
                                q_starts, q_lens)
         y = torch.empty(T, H * Dv, dtype=h.dtype, device=h.device)
         ops.head_rmsnorm_gate(y, o, self.norm_w, out_gate, self.eps,
-                              silu_gate=(kind == ops.SCAN_GLA))
+                              silu_gate=kind in (ops.SCAN_GLA,
+                                                 ops.SCAN_DELTA_HEAD))
         return ops.linear(y, self.w_o)
 
 

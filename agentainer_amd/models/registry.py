@@ -25,6 +25,10 @@ FAMILIES: Dict[str, Tuple[str, str, str, str]] = {
     # on the latent ones, convolution tails from the recurrent module
     "Sipelorn": ("agentainer_amd.models.sipelorn", "SIPELORN_CONFIGS",
                  "make_sipelorn_instance", "gated+masked+latent+recurrent"),
+    # latent attention, the delta-rule scan, sandwich norms on the gated
+    # family's residual kernel
+    "Mugazen": ("agentainer_amd.models.mugazen", "MUGAZEN_CONFIGS",
+                "make_mugazen_instance", "gated+latent+recurrent"),
 }
 
 

@@ -416,7 +416,7 @@ class GroupedSigmoidExperts(torch.nn.Module):
         self.n_gates = 1 if Fs > 0 else 0
         # fp32 router; the shared expert's gate is its last row
         self.router = _param(E + self.n_gates, width, dtype=f32)
-        self.correction = _param(E, dtype=f32)
+        self._route_params()
         # expert e owns rows [e*2F, e*2F+F) = gate, [e*2F+F, (e+1)*2F) = up;
         # then the shared expert's gate | up, then the caller's rows
         self.gu_rows = E * 2 * Fh + 2 * Fs
@@ -426,15 +426,32 @@ class GroupedSigmoidExperts(torch.nn.Module):
         # expert e owns columns [e*F, (e+1)*F); the shared expert the rest
         self.down = _param(width, E * Fh + Fs, dtype=dtype)
 
+    def _route_params(self):
+        self.correction = _param(self.fc.experts, dtype=torch.float32)
+
+    @torch.no_grad()
+    def _load_route(self, get):
+        rows = [get("router").float()]
+        if self.fc.shared_ff > 0:
+            rows.append(get("shared.sg").float().view(1, -1))
+        self.router.copy_(torch.cat(rows, dim=0))
+        self.correction.copy_(get("correction").float())
+
+    def route(self, h) -> torch.Tensor:
+        """Dense fp32 routing weights [T, E + n_gates], 0 = not chosen."""
+        fc = self.fc
+        logits = F.linear(h.float(), self.router)              # fp32 router
+        weight = torch.empty(h.size(0), fc.experts + self.n_gates,
+                             dtype=torch.float32, device=h.device)
+        return ops.grouped_sigmoid_route(
+            weight, logits, self.correction, fc.experts, fc.top, fc.groups,
+            fc.keep_groups, GROUP_TOP)
+
     @torch.no_grad()
     def load(self, get, extra=None):
         fc = self.fc
         E = fc.experts
-        rows = [get("router").float()]
-        if fc.shared_ff > 0:
-            rows.append(get("shared.sg").float().view(1, -1))
-        self.router.copy_(torch.cat(rows, dim=0))
-        self.correction.copy_(get("correction").float())
+        self._load_route(get)
         names = [f"e{e}." for e in range(E)]
         if fc.shared_ff > 0:
             names.append("shared.")
@@ -452,11 +469,7 @@ class GroupedSigmoidExperts(torch.nn.Module):
         steps are captured into a hipGraph)."""
         fc = self.fc
         T, E, Fh, Fs = h.size(0), fc.experts, fc.ff, fc.shared_ff
-        logits = F.linear(h.float(), self.router)              # fp32 router
-        weight = torch.empty(T, E + self.n_gates, dtype=torch.float32,
-                             device=h.device)
-        ops.grouped_sigmoid_route(weight, logits, self.correction, E, fc.top,
-                                  fc.groups, fc.keep_groups, GROUP_TOP)
+        weight = self.route(h)
         if allow_gather and T >= self.SPARSE_MIN_TOKENS and E > fc.top:
             return self._gathered(h, weight)
         gu = ops.linear(h, self.gate_up)

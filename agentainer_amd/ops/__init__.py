@@ -474,17 +474,21 @@ LATENT_SPLITS = int(os.environ.get("AGENTAINER_LATENT_SPLITS", "0"))
 
 def latent_window_attention(out, q_lat, cache, page_table, seq_lens,
                             query_starts, query_lens, scale: float,
-                            window: int, max_qlen: int = 1):
+                            window: int, max_qlen: int = 1, sink=None,
+                            head_gate=None):
+    """sink: fp32 [H], exp(sink_h) joins head h's denominator; head_gate
+    [T, H]: row t's head h is multiplied by sigmoid(head_gate[t, h])."""
     mod = _dispatch_latent("latent_window_attention", q_lat)
     if mod:
         mod.latent_window_attention(out, q_lat, cache, page_table, seq_lens,
                                     query_starts, query_lens, float(scale),
                                     int(window), int(max_qlen),
-                                    bool(LATENT_SIMPLE), int(LATENT_SPLITS))
+                                    bool(LATENT_SIMPLE), int(LATENT_SPLITS),
+                                    sink, head_gate)
     else:
         reference.latent_window_attention(out, q_lat, cache, page_table,
                                           seq_lens, query_starts, query_lens,
-                                          scale, window)
+                                          scale, window, sink, head_gate)
     return out
 
 
@@ -663,7 +667,7 @@ def masked_attention(out, q, k_cache, v_cache, page_table, seq_lens,
 # ---------------------------------------------------------------------
 # Post-norm residual with (1 + w) RMS norm, short causal convolutions with
 # a per-sequence tail, matrix-memory recurrences (gated linear attention,
-# gated delta rule, mLSTM) over per-sequence state, per-head output norm +
+# gated delta rules, mLSTM) over per-sequence state, per-head output norm +
 # gate, group-limited softmax routing and clamped gated experts. Own
 # extension (_hip_recurrent.so), same policy: required on a GPU, fp32
 # torch references on CPU.
@@ -713,6 +717,7 @@ def _dispatch_recurrent(name: str, t: torch.Tensor):
 SCAN_GLA = reference.SCAN_GLA
 SCAN_DELTA = reference.SCAN_DELTA
 SCAN_MLSTM = reference.SCAN_MLSTM
+SCAN_DELTA_HEAD = reference.SCAN_DELTA_HEAD
 
 
 def postln_rmsnorm_residual(x_res, y, w1p, eps: float, h_out,
@@ -798,6 +803,7 @@ def grouped_softmax_route(weight, logits, correction, top: int,
 
 def routed_clamped_glu(out, gu, weight, n_experts: int, limit: float,
                        slope: float):
+    """weight None: every expert weighs 1 (n_experts=1 is a dense unit)."""
     mod = _dispatch_recurrent("routed_clamped_glu", gu)
     if mod:
         mod.routed_clamped_glu(out, gu, weight, int(n_experts), float(limit),
@@ -808,7 +814,8 @@ def routed_clamped_glu(out, gu, weight, n_experts: int, limit: float,
 
 
 # ---------------------------------------------------------------------
-# Hashed bigram embedding, sigmoid-gated residual + layer norm, xIELU,
+# Hashed bigram embedding, learned-position embedding, sigmoid-gated or
+# unit-rms residual + layer or RMS norm, xIELU,
 # token-side gate, sigmoid group-limited routing, output-weighted gated
 # experts with a tail expert, latent rotary append, plain K/V append and
 # an elementwise output gate. Own extension (_hip_gated.so), same policy:
@@ -878,15 +885,50 @@ def bigram_embed(x_out, ids, embed, bigram, scale: float, mul_prev: int,
 
 
 def residual_update_norm(x_res, y, update: int, gate, gate_bias, rms_w,
-                         eps: float, norm_w, norm_b, h_out):
+                         eps: float, norm_w, norm_b, h_out,
+                         rms_norm: bool = False, add_rows=None,
+                         add_vec=None):
+    """rms_norm: h_out is the RMS norm of the stream instead of the layer
+    norm; add_rows [T, W] / add_vec [W] (fp32) join the stream after the
+    update and before the norm (see reference.residual_update_norm)."""
     mod = _dispatch_gated("residual_update_norm", x_res)
     if mod:
         mod.residual_update_norm(x_res, y, int(update), gate, gate_bias,
-                                 rms_w, float(eps), norm_w, norm_b, h_out)
+                                 rms_w, float(eps), norm_w, norm_b,
+                                 bool(rms_norm), add_rows, add_vec, h_out)
     else:
         reference.residual_update_norm(x_res, y, update, gate, gate_bias,
-                                       rms_w, eps, norm_w, norm_b, h_out)
+                                       rms_w, eps, norm_w, norm_b, h_out,
+                                       rms_norm, add_rows, add_vec)
     return h_out
+
+
+def position_embed_norm(x_out, ids, positions, embed, pos, scale: float, w,
+                        eps: float, x_copy=None):
+    """x_out (fp32) = rms_norm(scale * embed[id] + pos[position]) * w, also
+    into x_copy when given."""
+    mod = _dispatch_gated("position_embed_norm", x_out)
+    if mod:
+        mod.position_embed_norm(x_out, x_copy, ids, positions, embed, pos,
+                                float(scale), w, float(eps))
+    else:
+        reference.position_embed_norm(x_out, ids, positions, embed, pos,
+                                      scale, w, eps, x_copy)
+    return x_out
+
+
+def narrow_linear(x, w, bias=None):
+    """x [T, K] @ w [N, K]^T + bias with an fp32 result, for projections
+    whose few outputs are used in fp32 (routers, decays, write strengths).
+    bf16 operands on a GPU run the MFMA kernel; fp32 operands are an fp32
+    library product."""
+    if x.is_cuda and x.dtype == torch.bfloat16:
+        mod = _dispatch_gated("narrow_linear", x)
+        out = torch.empty(x.size(0), w.size(0), dtype=torch.float32,
+                          device=x.device)
+        mod.narrow_linear(out, x, w, bias)
+        return out
+    return torch.nn.functional.linear(x.float(), w.float(), bias)
 
 
 def xielu(out, z, coef):

@@ -61,14 +61,16 @@ RECURRENT_SOURCES = [
     "grouped_route.hip",
 ]
 
-# hashed bigram embedding, gated residual + layer norm, xIELU, sigmoid
-# group routing, output-weighted gated experts, latent rotary append
+# bigram / learned-position embeddings, gated residual + layer or RMS norm,
+# xIELU, sigmoid group routing, output-weighted gated experts, latent rotary
+# append, narrow projections with an fp32 result
 GATED_SOURCES = [
     "gated_bindings.cpp",
     "gated_norm.hip",
     "bigram_embed.hip",
     "sigmoid_route.hip",
     "latent_rotary.hip",
+    "narrow_linear.hip",
 ]
 
 SOURCES = [

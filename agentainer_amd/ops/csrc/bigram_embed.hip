@@ -1,4 +1,11 @@
-// Scaled token embedding plus a hashed bigram embedding (gfx950).
+// Token embeddings with a second table (gfx950).
+//
+// position_embed_norm: x[r] = rms_norm(scale * embed[id_r] + pos[p_r]) * w,
+// fp32 out, optionally written twice (the second copy is what later passes
+// of a repeated layer group add again). One workgroup per row; the sum stays
+// in registers between the two passes.
+//
+// bigram_embed: scaled token embedding plus a hashed bigram embedding
 //
 //   x[r] = scale * embed[id_r] + bigram[row_r]            (fp32 out)
 //   row_r = (mul_prev * id_(r-1) + mul_cur * id_r) mod buckets,
@@ -89,7 +96,82 @@ __global__ void bigram_state_kernel(int* __restrict__ prev_state,
   prev_state[slots[b]] = (int)ids[last];
 }
 
+constexpr int ROW_VALS = 32;   // values per thread: rows of up to 8192
+
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void position_embed_kernel(
+    float* __restrict__ x, float* __restrict__ x_copy,
+    const long* __restrict__ ids, const int* __restrict__ positions,
+    const T* __restrict__ embed, const T* __restrict__ pos, float scale,
+    const float* __restrict__ w, float eps, int W, long vocab, int n_pos) {
+  __shared__ float red[4];
+  const long r = blockIdx.x;
+  long id = ids[r];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  int p = positions[r];
+  p = p < 0 ? 0 : (p >= n_pos ? n_pos - 1 : p);
+  const T* er = embed + id * W;
+  const T* pr = pos + (long)p * W;
+  float v[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = k * 256 + threadIdx.x;
+    v[k] = i < W ? fmaf(ldf(er, i), scale, ldf(pr, i)) : 0.f;
+    ss = fmaf(v[k], v[k], ss);
+  }
+  const float rs = 1.0f / sqrtf(block_sum_256(ss, red) / (float)W + eps);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int i = k * 256 + threadIdx.x;
+    if (i < W) {
+      const float o = v[k] * rs * w[i];
+      x[r * W + i] = o;
+      if (x_copy) x_copy[r * W + i] = o;
+    }
+  }
+}
+
 }  // namespace
+
+void position_embed_norm(torch::Tensor x, c10::optional<torch::Tensor> x_copy,
+                         torch::Tensor ids, torch::Tensor positions,
+                         torch::Tensor embed, torch::Tensor pos, double scale,
+                         torch::Tensor w, double eps) {
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.is_contiguous() &&
+              x.dim() == 2);
+  const int T_ = x.size(0), W = x.size(1);
+  TORCH_CHECK(W <= 256 * ROW_VALS, "row wider than ", 256 * ROW_VALS);
+  TORCH_CHECK(ids.scalar_type() == at::kLong && ids.is_contiguous() &&
+              ids.numel() == T_);
+  TORCH_CHECK(positions.scalar_type() == at::kInt &&
+              positions.is_contiguous() && positions.numel() == T_);
+  TORCH_CHECK(embed.dim() == 2 && embed.is_contiguous() && embed.size(1) == W);
+  TORCH_CHECK(pos.dim() == 2 && pos.is_contiguous() && pos.size(1) == W &&
+              pos.size(0) >= 1 && pos.scalar_type() == embed.scalar_type());
+  TORCH_CHECK(w.scalar_type() == at::kFloat && w.is_contiguous() &&
+              w.numel() == W);
+  float* xc = nullptr;
+  if (x_copy.has_value()) {
+    TORCH_CHECK(x_copy->scalar_type() == at::kFloat &&
+                x_copy->is_contiguous() && x_copy->sizes() == x.sizes());
+    xc = x_copy->data_ptr<float>();
+  }
+  if (T_ == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+#define LAUNCH(N)                                                             \
+  hipLaunchKernelGGL((position_embed_kernel<T, N>), dim3(T_), dim3(256), 0,   \
+                     stream, x.data_ptr<float>(), xc, ids.data_ptr<long>(),   \
+                     positions.data_ptr<int>(), (const T*)embed.data_ptr(),   \
+                     (const T*)pos.data_ptr(), (float)scale,                  \
+                     w.data_ptr<float>(), (float)eps, W, (long)embed.size(0), \
+                     (int)pos.size(0))
+  LATENT_DISPATCH_T(embed, {
+    if (W <= 256 * 8) LAUNCH(8);
+    else LAUNCH(ROW_VALS);
+  });
+#undef LAUNCH
+}
 
 void bigram_embed(torch::Tensor x, torch::Tensor ids, torch::Tensor embed,
                   c10::optional<torch::Tensor> bigram, double scale,

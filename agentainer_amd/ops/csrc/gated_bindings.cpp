@@ -1,6 +1,7 @@
-// pybind11 bindings: hashed bigram embedding, gated residual + layer norm,
-// xIELU, token-side gate, sigmoid group-limited routing, output-weighted
-// gated experts, latent rotary append, plain K/V append, output gate.
+// pybind11 bindings: hashed bigram embedding, learned-position embedding,
+// gated residual + layer or RMS norm, xIELU, token-side gate, sigmoid group-limited routing, output-weighted
+// gated experts, latent rotary append, plain K/V append, output gate,
+// narrow projections with an fp32 result.
 #include <torch/extension.h>
 
 using OptT = c10::optional<torch::Tensor>;
@@ -11,7 +12,14 @@ void bigram_embed(torch::Tensor x, torch::Tensor ids, torch::Tensor embed,
                   torch::Tensor seq_lens, OptT query_starts, OptT query_lens);
 void residual_update_norm(torch::Tensor x, OptT y, long update, OptT gate,
                           OptT gate_bias, OptT rms_w, double eps, OptT norm_w,
-                          OptT norm_b, OptT h);
+                          OptT norm_b, bool rms_norm, OptT add_rows,
+                          OptT add_vec, OptT h);
+void position_embed_norm(torch::Tensor x, OptT x_copy, torch::Tensor ids,
+                         torch::Tensor positions, torch::Tensor embed,
+                         torch::Tensor pos, double scale, torch::Tensor w,
+                         double eps);
+void narrow_linear(torch::Tensor out, torch::Tensor x, torch::Tensor w,
+                   OptT bias);
 void xielu(torch::Tensor out, torch::Tensor z, torch::Tensor coef);
 void gelu_gate_rows(torch::Tensor out, torch::Tensor t, torch::Tensor table,
                     torch::Tensor ids, long col0);
@@ -34,7 +42,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("bigram_embed", &bigram_embed,
         "scaled embedding + hashed bigram row; previous token kept as state");
   m.def("residual_update_norm", &residual_update_norm,
-        "gated / unit-rms fp32 residual update fused with a layer norm");
+        "gated / unit-rms fp32 residual update fused with a layer / RMS norm");
+  m.def("position_embed_norm", &position_embed_norm,
+        "RMS norm of scale * embedding + learned position row");
+  m.def("narrow_linear", &narrow_linear,
+        "bf16 rows times a narrow bf16 weight, fp32 result");
   m.def("xielu", &xielu, "xIELU activation");
   m.def("gelu_gate_rows", &gelu_gate_rows,
         "gelu_tanh(t) * table[id] column slice");

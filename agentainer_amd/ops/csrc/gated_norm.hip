@@ -1,13 +1,16 @@
-// Gated residual update fused with a layer norm, and the elementwise
+// Gated residual update fused with a layer or RMS norm, and the elementwise
 // activations of the gated family (gfx950).
 //
 //   residual_update_norm   x (fp32, in place) gets one of
 //                            nothing
 //                            x += sigmoid(gate + gate_bias) * y
 //                            x += y / sqrt(mean(y^2) + eps) * rms_w
+//                          then optionally x += add_rows[row] + add_vec (what
+//                          a repeated group of layers takes in before a pass),
 //                          and then h = ((x - mean) / sqrt(var + eps)) * w + b
-//                          in the compute dtype (the next GEMM's input), or
-//                          h = x cast (no norm weights), or nothing.
+//                          or, as an RMS norm, h = x / sqrt(mean(x^2) + eps) *
+//                          w + b in the compute dtype (the next GEMM's input),
+//                          or h = x cast (no norm weights), or nothing.
 //                          One 256-thread workgroup per row; the updated row
 //                          stays in registers between the passes (rows up to
 //                          256 * 4 * ROW_REGS values), so x is read and
@@ -57,7 +60,8 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
     const T* __restrict__ gate, long g_rs, const float* __restrict__ gate_bias,
     const float* __restrict__ rms_w, float eps,
     const float* __restrict__ norm_w, const float* __restrict__ norm_b,
-    T* __restrict__ h, int W) {
+    bool rms_norm, const float* __restrict__ add_rows,
+    const float* __restrict__ add_vec, T* __restrict__ h, int W) {
   __shared__ float red[4];
   const long row = blockIdx.x;
   float* xr = x + row * W;
@@ -107,7 +111,20 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
         for (int j = 0; j < VEC; ++j)
           xv[k][j] = fmaf(v[j] * scale_y, w[j], xv[k][j]);
       }
-      if (update != UPD_NONE) stv<float, VEC>(xr, i, xv[k]);
+      if (add_rows) {
+        float v[VEC];
+        ldv<float, VEC>(add_rows + row * W, i, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) xv[k][j] += v[j];
+      }
+      if (add_vec) {
+        float v[VEC];
+        ldv<float, VEC>(add_vec, i, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) xv[k][j] += v[j];
+      }
+      if (update != UPD_NONE || add_rows || add_vec)
+        stv<float, VEC>(xr, i, xv[k]);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) sum += xv[k][j];
     }
@@ -122,7 +139,7 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
     }
     return;
   }
-  const float mean = block_sum_256(sum, red) * inv_w;
+  const float mean = rms_norm ? 0.f : block_sum_256(sum, red) * inv_w;
   float sq = 0.f;
 #pragma unroll
   for (int k = 0; k < NREG; ++k) {
@@ -238,7 +255,9 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
                           c10::optional<torch::Tensor> gate_bias,
                           c10::optional<torch::Tensor> rms_w, double eps,
                           c10::optional<torch::Tensor> norm_w,
-                          c10::optional<torch::Tensor> norm_b,
+                          c10::optional<torch::Tensor> norm_b, bool rms_norm,
+                          c10::optional<torch::Tensor> add_rows,
+                          c10::optional<torch::Tensor> add_vec,
                           c10::optional<torch::Tensor> h) {
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.is_contiguous() &&
               x.dim() == 2);
@@ -254,6 +273,11 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
   check_vec(rms_w);
   check_vec(norm_w);
   check_vec(norm_b);
+  check_vec(add_vec);
+  if (add_rows.has_value())
+    TORCH_CHECK(add_rows->scalar_type() == at::kFloat &&
+                add_rows->is_contiguous() && add_rows->dim() == 2 &&
+                add_rows->size(0) == rows && add_rows->size(1) == W);
   bool vec = W % 4 == 0;
   long y_rs = 0, g_rs = 0;
   at::ScalarType ct = at::kFloat;
@@ -284,21 +308,23 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
   } else {
     TORCH_CHECK(!norm_w.has_value());
   }
-  if (rows == 0 || (update == UPD_NONE && !h.has_value())) return;
-  if (!have_ct) return;
+  const bool adds = add_rows.has_value() || add_vec.has_value();
+  if (rows == 0 || (update == UPD_NONE && !adds && !h.has_value())) return;
   const void* yp = update != UPD_NONE ? y->data_ptr() : nullptr;
   const void* gp = update == UPD_GATE ? gate->data_ptr() : nullptr;
   const float* gb = gate_bias.has_value() ? gate_bias->data_ptr<float>() : nullptr;
   const float* rw = rms_w.has_value() ? rms_w->data_ptr<float>() : nullptr;
   const float* nw = norm_w.has_value() ? norm_w->data_ptr<float>() : nullptr;
   const float* nb = norm_b.has_value() ? norm_b->data_ptr<float>() : nullptr;
+  const float* ar = add_rows.has_value() ? add_rows->data_ptr<float>() : nullptr;
+  const float* av = add_vec.has_value() ? add_vec->data_ptr<float>() : nullptr;
   void* hp = h.has_value() ? h->data_ptr() : nullptr;
   auto stream = at::hip::getCurrentHIPStream();
 #define LAUNCH(TT, V, N)                                                      \
   hipLaunchKernelGGL((residual_update_norm_kernel<TT, V, N>), dim3(rows),     \
                      dim3(256), 0, stream, x.data_ptr<float>(),               \
                      (const TT*)yp, y_rs, (int)update, (const TT*)gp, g_rs,   \
-                     gb, rw, (float)eps, nw, nb, (TT*)hp, W)
+                     gb, rw, (float)eps, nw, nb, rms_norm, ar, av, (TT*)hp, W)
   const bool bf = ct == at::kBFloat16;
   TORCH_CHECK(bf || ct == at::kFloat, "expected bf16 or fp32 rows");
   if (vec) {

@@ -12,7 +12,8 @@
 //     input row scales its output): g = min(gate, limit),
 //     u = clamp(up, -limit, limit),
 //     out[t, e, f] = w[t, e] * g * sigmoid(slope * g) * (u + 1); experts
-//     with w == 0 write 0 without reading their columns.
+//     with w == 0 write 0 without reading their columns. Without a weight
+//     every w is 1 (a dense unit is one unweighted expert).
 
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
@@ -131,7 +132,7 @@ __global__ void clamped_glu_kernel(T* __restrict__ out,
   const long t = i / ((long)E * F);
   const int rem = (int)(i % ((long)E * F));
   const int e = rem / F, f = rem % F;
-  const float w = weight[t * w_rs + e];
+  const float w = weight ? weight[t * w_rs + e] : 1.0f;
   float o[VEC];
   if (w == 0.f) {
 #pragma unroll
@@ -190,15 +191,21 @@ void grouped_softmax_route(torch::Tensor weight, torch::Tensor logits,
 }
 
 void routed_clamped_glu(torch::Tensor out, torch::Tensor gu,
-                        torch::Tensor weight, long n_experts, double limit,
-                        double slope) {
+                        c10::optional<torch::Tensor> weight, long n_experts,
+                        double limit, double slope) {
   TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && gu.dim() == 2 &&
               gu.stride(1) == 1 && gu.scalar_type() == out.scalar_type());
-  TORCH_CHECK(weight.scalar_type() == at::kFloat && weight.dim() == 2 &&
-              weight.stride(1) == 1);
   const int T_ = out.size(0), E = n_experts;
-  TORCH_CHECK(E >= 1 && weight.size(1) >= E && weight.size(0) == T_ &&
-              gu.size(0) == T_);
+  TORCH_CHECK(E >= 1 && gu.size(0) == T_);
+  const float* wp = nullptr;
+  long w_rs = 0;
+  if (weight.has_value()) {
+    TORCH_CHECK(weight->scalar_type() == at::kFloat && weight->dim() == 2 &&
+                weight->stride(1) == 1 && weight->size(1) >= E &&
+                weight->size(0) == T_);
+    wp = weight->data_ptr<float>();
+    w_rs = weight->stride(0);
+  }
   TORCH_CHECK(out.size(1) % E == 0);
   const int F = out.size(1) / E;
   TORCH_CHECK(gu.size(1) == (long)2 * E * F, "gate|up width mismatch");
@@ -211,14 +218,12 @@ void routed_clamped_glu(torch::Tensor out, torch::Tensor gu,
     if (vec) {
       hipLaunchKernelGGL((clamped_glu_kernel<T, 4>), dim3((n / 4 + 255) / 256),
                          dim3(256), 0, stream, (T*)out.data_ptr(),
-                         (const T*)gu.data_ptr(), weight.data_ptr<float>(),
-                         (long)weight.stride(0), n, E, F, (long)gu.stride(0),
+                         (const T*)gu.data_ptr(), wp, w_rs, n, E, F, (long)gu.stride(0),
                          (float)limit, (float)slope);
     } else {
       hipLaunchKernelGGL((clamped_glu_kernel<T, 1>), dim3((n + 255) / 256),
                          dim3(256), 0, stream, (T*)out.data_ptr(),
-                         (const T*)gu.data_ptr(), weight.data_ptr<float>(),
-                         (long)weight.stride(0), n, E, F, (long)gu.stride(0),
+                         (const T*)gu.data_ptr(), wp, w_rs, n, E, F, (long)gu.stride(0),
                          (float)limit, (float)slope);
     }
   });

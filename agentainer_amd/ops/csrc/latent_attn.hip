@@ -9,7 +9,10 @@
 //   s[h,t,j]   = scale * <q_lat[h,t], c[j]>      for  pos(t)-window < j <= pos(t)
 //   o_lat[h,t] = sum_j softmax_j(s[h,t,:]) c[j]
 //
-// Scores, softmax and the accumulation are fp32.
+// Scores, softmax and the accumulation are fp32. Two optional parts, both
+// applied where the sum is normalized: a SINK per head (exp(sink_h) joins
+// the denominator once, unscaled, with no key and no value) and a HEAD GATE
+// (row t's head h is multiplied by sigmoid(gate[t, h])).
 //
 // Kernels:
 //   latent_norm_append    RMS-norm the query latent and the kv latent held in
@@ -42,6 +45,30 @@
 namespace {
 
 typedef __bf16 bf16v8 __attribute__((ext_vector_type(8)));
+
+// optional sink and gate of the finished sum; either pointer may be null
+template <typename T>
+struct HeadTail {
+  const float* sink;   // [H]
+  const T* gate;       // [T, H], row stride gate_rs
+  long gate_rs;
+
+  // factor that turns an unnormalized sum with running maximum m and
+  // exponential mass l into the head's output
+  __device__ __forceinline__ float factor(float m, float l, int h,
+                                          long row) const {
+    float f = 1.0f;
+    if (sink) {
+      const float s = sink[h];
+      const float mn = fmaxf(m, s);
+      f = (m == -FLT_MAX) ? 0.f : expf(m - mn);
+      l = l * f + expf(s - mn);
+    }
+    f = l > 0.f ? f / l : 0.f;
+    if (gate) f = f / (1.0f + expf(-ldf(gate, row * gate_rs + h)));
+    return f;
+  }
+};
 
 // ------------------------------------------------------------------
 // latent_norm_append
@@ -89,7 +116,8 @@ __global__ __launch_bounds__(64) void latent_attn_rowwave_kernel(
     long o_hs, long o_ts, const T* __restrict__ cache,
     const int* __restrict__ page_table, const int* __restrict__ seq_lens,
     const int* __restrict__ q_starts, const int* __restrict__ q_lens,
-    float scale, int window, int Rp, int PS, int max_pages) {
+    float scale, int window, int Rp, int PS, int max_pages,
+    const HeadTail<T> tail) {
   extern __shared__ float smem[];
   float* q_s = smem;        // [Rp]
   float* p_s = smem + Rp;   // [64]
@@ -156,7 +184,7 @@ __global__ __launch_bounds__(64) void latent_attn_rowwave_kernel(
     }
     __syncthreads();
   }
-  const float inv = 1.0f / l;
+  const float inv = tail.factor(m, l, h, rowi);
 #pragma unroll
   for (int k = 0; k < RW_MAX_ACC; ++k) {
     const int d = k * WAVE + lane;
@@ -182,7 +210,8 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(
     const int* __restrict__ page_table, const int* __restrict__ seq_lens,
     const int* __restrict__ q_starts, const int* __restrict__ q_lens,
     float scale, int window, int H, int nc, int PS, int max_pages,
-    float* __restrict__ part_o, float* __restrict__ part_ml, int n_splits) {
+    float* __restrict__ part_o, float* __restrict__ part_ml, int n_splits,
+    const HeadTail<short> tail) {
   extern __shared__ __attribute__((aligned(16))) short lds[];
   const int Rp = nc * 32;
   const int KS = Rp + 8;                       // padded row-major stride
@@ -402,7 +431,8 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(
   for (int r = 0; r < 4; ++r) {
     const int rr = rw0 + lg * 4 + r;
     if (rr >= nrows) continue;
-    const float inv = l_run[r] > 0.f ? 1.0f / l_run[r] : 0.f;
+    const float inv =
+        tail.factor(m_run[r], l_run[r], rr % H, row_base + rr / H);
     short* op = out + (rr % H) * o_hs + (row_base + rr / H) * o_ts;
 #pragma unroll
     for (int dt = 0; dt < 2 * MAXNC; ++dt)
@@ -614,7 +644,8 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(
 __global__ __launch_bounds__(128) void latent_attn_combine_kernel(
     short* __restrict__ out, long o_hs, long o_ts,
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
-    const int* __restrict__ seq_lens, int H, int Rp, int n_splits) {
+    const int* __restrict__ seq_lens, int H, int Rp, int n_splits,
+    const HeadTail<short> tail) {
   const int h = blockIdx.x, b = blockIdx.y;
   short* op = out + h * o_hs + (long)b * o_ts;
   if (seq_lens[b] <= 0) {
@@ -630,7 +661,7 @@ __global__ __launch_bounds__(128) void latent_attn_combine_kernel(
     const float m = part_ml[pr * 2];
     if (m != -FLT_MAX) L += part_ml[pr * 2 + 1] * __expf(m - M);
   }
-  const float inv = L > 0.f ? 1.0f / L : 0.f;
+  const float inv = tail.factor(M, L, h, b);
   // Rp is a multiple of 32: 4 consecutive columns per thread
   for (int d = threadIdx.x * 4; d < Rp; d += 128 * 4) {
     float acc[4] = {0.f, 0.f, 0.f, 0.f};
@@ -725,7 +756,9 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                              c10::optional<torch::Tensor> query_starts,
                              c10::optional<torch::Tensor> query_lens,
                              double scale, long window, long max_qlen,
-                             bool force_simple, long splits) {
+                             bool force_simple, long splits,
+                             c10::optional<torch::Tensor> sink,
+                             c10::optional<torch::Tensor> head_gate) {
   // splits < 0: run decode on the tile kernel with -splits slices (A/B)
   const bool force_tile_decode = splits < 0;
   if (splits < 0) splits = -splits;
@@ -758,6 +791,24 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
     max_qlen = 1;
   }
   TORCH_CHECK(window >= 1 && max_qlen >= 1);
+  const float* sink_p = nullptr;
+  if (sink.has_value()) {
+    TORCH_CHECK(sink->scalar_type() == at::kFloat && sink->is_contiguous() &&
+                sink->numel() == H, "sink must be fp32, one per head");
+    sink_p = sink->data_ptr<float>();
+  }
+  const void* gate_p = nullptr;
+  long gate_rs = 0;
+  if (head_gate.has_value()) {
+    TORCH_CHECK(head_gate->scalar_type() == cache.scalar_type() &&
+                head_gate->dim() == 2 && head_gate->size(0) == Tq &&
+                head_gate->size(1) == H &&
+                (H == 1 || head_gate->stride(1) == 1),
+                "head gate must be [rows, heads] in the compute dtype");
+    gate_p = head_gate->data_ptr();
+    gate_rs = head_gate->stride(0);
+  }
+  const HeadTail<short> tail{sink_p, (const short*)gate_p, gate_rs};
   if (B == 0 || Tq == 0) return;
   const int max_pages = page_table.size(1);
   auto stream = at::hip::getCurrentHIPStream();
@@ -799,7 +850,7 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                          stream, (short*)out.data_ptr(), (long)out.stride(0),
                          (long)out.stride(1), part_o.data_ptr<float>(),
                          part_ml.data_ptr<float>(), seq_lens.data_ptr<int>(),
-                         H, Rp, (int)ns);
+                         H, Rp, (int)ns, tail);
       return;
     }
     const long rows = max_qlen * H;
@@ -845,7 +896,7 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                        max_pages,                                              \
                        n_splits > 0 ? part_o.data_ptr<float>() : nullptr,      \
                        n_splits > 0 ? part_ml.data_ptr<float>() : nullptr,     \
-                       n_splits);                                              \
+                       n_splits, tail);                                        \
   } while (0)
     if (nc <= 2) LA_LAUNCH(2);
     else if (nc <= 4) LA_LAUNCH(4);
@@ -857,7 +908,7 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                          stream, (short*)out.data_ptr(), (long)out.stride(0),
                          (long)out.stride(1), part_o.data_ptr<float>(),
                          part_ml.data_ptr<float>(), seq_lens.data_ptr<int>(),
-                         H, Rp, n_splits);
+                         H, Rp, n_splits, tail);
     if (launched) return;
   }
   TORCH_CHECK(Rp <= WAVE * RW_MAX_ACC, "latent rank too large");
@@ -870,7 +921,8 @@ void latent_window_attention(torch::Tensor out, torch::Tensor q_lat,
                        (long)out.stride(0), (long)out.stride(1),
                        (const T*)cache.data_ptr(), page_table.data_ptr<int>(),
                        seq_lens.data_ptr<int>(), qs, ql, (float)scale,
-                       (int)window, Rp, PS, max_pages);
+                       (int)window, Rp, PS, max_pages,
+                       HeadTail<T>{sink_p, (const T*)gate_p, gate_rs});
   });
 }
 

@@ -1,13 +1,15 @@
 // Matrix-memory recurrences over per-sequence state (gfx950): gated linear
-// attention, gated delta rule with per-key-channel decay, and the mLSTM
+// attention, gated delta rule with per-key-channel decay or with one decay
+// per head, and the mLSTM
 // memory with a running-maximum stabilizer — plus the per-head output norm
 // and gate that follow them.
 //
 // Per head the memory S has `D` key rows and `Dv` value columns; every
 // column evolves on its own given the token's k, q and decays:
 //
-//   S'   = g (.) S                      (g: per key row; mLSTM: one number)
-//   a1_j = sum_r S'[r, j] k[r]          (delta rule only)
+//   S'   = g (.) S                      (g: per key row; mLSTM and the
+//                                        head-decay delta rule: one number)
+//   a1_j = sum_r S'[r, j] k[r]          (delta rules only)
 //   a2_j = sum_r S'[r, j] q[r]
 //   u_j  = beta (v_j - a1_j)  |  v_j  |  e^(i - m') v_j
 //   S    = S' + k u^T,   o_j = a2_j + u_j (k . q)     [= (S^T q)_j]
@@ -26,7 +28,8 @@
 // Tokens are processed strictly in order, eight at a time: the raw inputs
 // of the NEXT eight tokens are loaded into registers while the current
 // eight are computed. The per-channel decays (sigmoid / softplus / exp) are
-// evaluated beforehand by a fully parallel pass, the mLSTM gates and the
+// evaluated beforehand by a fully parallel pass, one-number decays while
+// their token is staged, the mLSTM gates and the
 // running maximum by one wave per chunk (lane c: token c) — the serial
 // loop holds multiply-adds only. Prompt portions and single decoded tokens
 // run the same code, so a position's result does not depend on where the
@@ -41,6 +44,8 @@ namespace mm {
 void launch_gla(const ScanArgs& a, int B, int lanes, bool bf16, hipStream_t s);
 void launch_delta(const ScanArgs& a, int B, int lanes, bool bf16,
                   hipStream_t s);
+void launch_delta_head(const ScanArgs& a, int B, int lanes, bool bf16,
+                       hipStream_t s);
 void launch_mlstm(const ScanArgs& a, int B, int lanes, bool bf16,
                   hipStream_t s);
 }  // namespace mm
@@ -49,6 +54,7 @@ namespace {
 
 using mm::KIND_GLA;
 using mm::KIND_DELTA;
+using mm::KIND_DELTA_HEAD;
 using mm::KIND_MLSTM;
 using mm::ScanArgs;
 
@@ -142,7 +148,7 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
                         torch::Tensor state_slots, torch::Tensor seq_lens,
                         c10::optional<torch::Tensor> query_starts,
                         c10::optional<torch::Tensor> query_lens, long lanes) {
-  TORCH_CHECK(kind >= 0 && kind <= 2, "unknown recurrence");
+  TORCH_CHECK(kind >= 0 && kind <= 3, "unknown recurrence");
   TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 && out.dim() == 3);
   const int T_ = v.size(0), H = v.size(1), Dv = v.size(2);
   const int G = k.size(1), D = k.size(2);
@@ -177,16 +183,19 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
     TORCH_CHECK(G == H);
     a.n_state = n_state->data_ptr<float>();
     a.m_state = m_state->data_ptr<float>();
+  } else if (kind == KIND_DELTA_HEAD) {
+    TORCH_CHECK(gate.size(1) == H && gate_bias->numel() == H);
   } else {
     TORCH_CHECK(gate.size(1) == (long)H * D && gate_bias->numel() == (long)H * D);
   }
-  if (kind == KIND_DELTA) {
+  if (mm::is_delta(kind)) {
     TORCH_CHECK(head_rate.has_value() && beta.has_value());
     TORCH_CHECK(head_rate->scalar_type() == at::kFloat &&
                 head_rate->is_contiguous() && head_rate->numel() == H);
     TORCH_CHECK(beta->scalar_type() == at::kFloat && beta->dim() == 2 &&
                 beta->size(0) == T_ && beta->size(1) == H &&
                 beta->stride(1) == 1);
+    a.head_rate = head_rate->data_ptr<float>();
     a.beta = beta->data_ptr<float>();
     a.beta_rs = beta->stride(0);
   }
@@ -214,7 +223,7 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
   a.gate_bias = gate_bias->data_ptr<float>();
   auto stream = at::hip::getCurrentHIPStream();
   torch::Tensor decay;
-  if (kind != KIND_MLSTM) {
+  if (mm::channel_decay(kind)) {
     decay = torch::empty({T_, (long)H * D}, S.options());
     const long n = (long)T_ * H * D;
     if (kind == KIND_GLA) {
@@ -250,6 +259,8 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
               "expected bf16 or fp32 q, k, v");
   if (kind == KIND_GLA) mm::launch_gla(a, B, (int)lanes, bf16, stream);
   else if (kind == KIND_DELTA) mm::launch_delta(a, B, (int)lanes, bf16, stream);
+  else if (kind == KIND_DELTA_HEAD)
+    mm::launch_delta_head(a, B, (int)lanes, bf16, stream);
   else mm::launch_mlstm(a, B, (int)lanes, bf16, stream);
   if (kind == KIND_MLSTM) {
     hipLaunchKernelGGL(scatter_nm_kernel, dim3((H * D + 255) / 256, B),

@@ -8,7 +8,15 @@
 
 namespace mm {
 
-constexpr int KIND_GLA = 0, KIND_DELTA = 1, KIND_MLSTM = 2;
+constexpr int KIND_GLA = 0, KIND_DELTA = 1, KIND_MLSTM = 2, KIND_DELTA_HEAD = 3;
+// delta rules correct the memory towards v; the other kinds add k v^T
+constexpr bool is_delta(int kind) {
+  return kind == KIND_DELTA || kind == KIND_DELTA_HEAD;
+}
+// decays per key channel (staged vectors) or one number per head and token
+constexpr bool channel_decay(int kind) {
+  return kind == KIND_GLA || kind == KIND_DELTA;
+}
 constexpr int CH = 8;      // tokens staged together
 constexpr int WAVES = 4;   // waves of a workgroup; they share the staging
 constexpr int TPW = CH / WAVES;
@@ -19,8 +27,10 @@ struct ScanArgs {
   const void* k;
   const void* v;         // [T, H, Dv]
   const float* gate;     // gla / delta: decays [T, H*D], already evaluated;
-                         // mLSTM: gate pre-activations [T, 2H]
+                         // mLSTM: gate pre-activations [T, 2H];
+                         // head delta: decay pre-activations [T, H]
   const float* gate_bias;
+  const float* head_rate;  // [H] (head delta)
   const float* beta;     // [T, H], row stride beta_rs
   float* S;              // [slots, H, Dv, D]
   const float* n_state;  // [slots, H, D]   (read at the start)
@@ -78,8 +88,8 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
   constexpr int R4 = RPT / 4;
   __shared__ __attribute__((aligned(16))) float kbuf[CH][ROWS];
   __shared__ __attribute__((aligned(16))) float qbuf[CH][ROWS];
-  __shared__ __attribute__((aligned(16))) float gbuf[KIND == KIND_MLSTM ? 1 : CH][ROWS];
-  __shared__ float sc[CH][4];   // k.q | write scale (beta, e^(i-m)) | e^(f+m-m') | e^(-m')
+  __shared__ __attribute__((aligned(16))) float gbuf[channel_decay(KIND) ? CH : 1][ROWS];
+  __shared__ float sc[CH][4];   // k.q | write scale (beta, e^(i-m)) | one-number decay | e^(-m')
 
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int col = lane / NSUB, sub = lane % NSUB;
@@ -132,8 +142,8 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
   // tokens c = w, w + WAVES, ... of a chunk for the whole workgroup; every
   // lane keeps its own column's v; wave 0 evaluates the mLSTM gates, lane
   // c those of token c.
-  float rk[TPW][EPL], rq[TPW][EPL], rg[KIND == KIND_MLSTM ? 1 : TPW][EPL];
-  float rb[TPW];
+  float rk[TPW][EPL], rq[TPW][EPL], rg[channel_decay(KIND) ? TPW : 1][EPL];
+  float rb[TPW], rz[KIND == KIND_DELTA_HEAD ? TPW : 1];
   float rv[CH];
   float rgi = 0.f, rgf = 0.f;
   const TI* qp = (const TI*)a.q;
@@ -153,10 +163,12 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           const int rc = ok ? r : 0;
           rk[i][e] = ok ? ldf(kp, row * a.k_rs + (long)g * D + rc) : 0.f;
           rq[i][e] = ok ? ldf(qp, row * a.q_rs + (long)g * D + rc) : 0.f;
-          if constexpr (KIND != KIND_MLSTM)
+          if constexpr (channel_decay(KIND))
             rg[i][e] = ok ? a.gate[row * a.gate_rs + (long)h * D + rc] : 1.f;
         }
-        if constexpr (KIND == KIND_DELTA) rb[i] = a.beta[row * a.beta_rs + h];
+        if constexpr (is_delta(KIND)) rb[i] = a.beta[row * a.beta_rs + h];
+        if constexpr (KIND == KIND_DELTA_HEAD)
+          rz[i] = a.gate[row * a.gate_rs + h];
       }
     }
 #pragma unroll
@@ -173,6 +185,11 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
   };
 
   float bias_i = 0.f, bias_f = 0.f;
+  float rate = 0.f;
+  if constexpr (KIND == KIND_DELTA_HEAD) {
+    bias_i = a.gate_bias[h];
+    rate = expf(a.head_rate[h]);
+  }
   if constexpr (KIND == KIND_MLSTM) {
     bias_i = a.gate_bias[h];
     bias_f = a.gate_bias[H + h];
@@ -196,14 +213,16 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           if (r < ROWS) {
             kbuf[c][r] = kk;
             qbuf[c][r] = qq;
-            if constexpr (KIND != KIND_MLSTM) gbuf[c][r] = rg[i][e];
+            if constexpr (channel_decay(KIND)) gbuf[c][r] = rg[i][e];
           }
         }
         kq = wave_total(kq);
         if (lane == 0) {
           sc[c][0] = kq;
-          if constexpr (KIND == KIND_DELTA)
+          if constexpr (is_delta(KIND))
             sc[c][1] = 1.0f / (1.0f + expf(-rb[i]));
+          if constexpr (KIND == KIND_DELTA_HEAD)
+            sc[c][2] = expf(-rate * soft_plus(rz[i] + bias_i));
         }
       }
     }
@@ -236,7 +255,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
       cv[c] = rv[c];
       ckq[c] = sc[c][0];
       cu[c] = KIND == KIND_GLA ? 1.f : sc[c][1];
-      cdf[c] = KIND == KIND_MLSTM ? sc[c][2] : 1.f;
+      cdf[c] = channel_decay(KIND) ? 1.f : sc[c][2];
       cei[c] = KIND == KIND_MLSTM ? sc[c][3] : 0.f;
     }
     if (t0 + CH < n_tok) load_chunk(t0 + CH);    // lands during the compute
@@ -255,7 +274,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           const float4 k4 = *reinterpret_cast<const float4*>(&kbuf[c][r]);
           const float4 q4 = *reinterpret_cast<const float4*>(&qbuf[c][r]);
           float4 g4;
-          if constexpr (KIND == KIND_MLSTM) {
+          if constexpr (!channel_decay(KIND)) {
             g4 = make_float4(cdf[c], cdf[c], cdf[c], cdf[c]);
           } else {
             g4 = *reinterpret_cast<const float4*>(&gbuf[c][r]);
@@ -267,7 +286,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           for (int e = 0; e < 4; ++e) {
             const float s = S[i4 * 4 + e] * gg[e];
             S[i4 * 4 + e] = s;
-            if constexpr (KIND == KIND_DELTA) a1[e] = fmaf(s, kk[e], a1[e]);
+            if constexpr (is_delta(KIND)) a1[e] = fmaf(s, kk[e], a1[e]);
             a2[e] = fmaf(s, qq[e], a2[e]);
             if constexpr (KIND == KIND_MLSTM) {
               const float nn = fmaf(nst[i4 * 4 + e], cdf[c], cu[c] * kk[e]);
@@ -278,7 +297,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         }
         const float a2s = sub_sum<NSUB>((a2[0] + a2[1]) + (a2[2] + a2[3]));
         float u;
-        if constexpr (KIND == KIND_DELTA) {
+        if constexpr (is_delta(KIND)) {
           const float a1s = sub_sum<NSUB>((a1[0] + a1[1]) + (a1[2] + a1[3]));
           u = cu[c] * (cv[c] - a1s);
         } else if constexpr (KIND == KIND_MLSTM) {

@@ -26,9 +26,8 @@ void head_rmsnorm_gate(torch::Tensor out, torch::Tensor o, torch::Tensor w,
 void grouped_softmax_route(torch::Tensor weight, torch::Tensor logits,
                            OptT correction, long top, long n_groups,
                            long keep_groups, double scale);
-void routed_clamped_glu(torch::Tensor out, torch::Tensor gu,
-                        torch::Tensor weight, long n_experts, double limit,
-                        double slope);
+void routed_clamped_glu(torch::Tensor out, torch::Tensor gu, OptT weight,
+                        long n_experts, double limit, double slope);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "agentainer_amd CDNA4 (gfx950) recurrent-family kernels";
@@ -37,7 +36,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("short_conv_state", &short_conv_state,
         "depthwise causal convolution with a per-sequence tail");
   m.def("matrix_memory_scan", &matrix_memory_scan,
-        "gated linear attention / gated delta rule / mLSTM over state");
+        "gated linear attention / gated delta rules / mLSTM over state");
   m.def("head_rmsnorm_gate", &head_rmsnorm_gate,
         "per-head RMS norm, weight and output gate");
   m.def("grouped_softmax_route", &grouped_softmax_route,

@@ -236,13 +236,16 @@ def latent_norm_append(proj: torch.Tensor, q_off: int, q_rank: int,
 def latent_window_attention(out: torch.Tensor, q_lat: torch.Tensor,
                             cache: torch.Tensor, page_table: torch.Tensor,
                             seq_lens: torch.Tensor, query_starts,
-                            query_lens, scale: float, window: int) -> None:
+                            query_lens, scale: float, window: int,
+                            sink=None, head_gate=None) -> None:
     """Multi-query attention in latent space: every head's query q_lat[h, t]
     (already mapped into the latent basis) scores the cached latents
     themselves, and the output is the softmax-weighted sum of the same
     latents. A query at position p sees keys at p - window < j <= p.
     q_lat/out: [H, T, Rp]; cache [P, PS, Rp]. query_starts/query_lens None
-    means one new token per sequence (decode)."""
+    means one new token per sequence (decode). sink [H]: exp(sink_h) joins
+    head h's softmax denominator, with no key and no value; head_gate [T, H]:
+    the output is multiplied by sigmoid(head_gate[t, h])."""
     H = q_lat.size(0)
     PS, Rp = cache.size(1), cache.size(2)
     flat = cache.view(-1, Rp)
@@ -266,9 +269,15 @@ def latent_window_attention(out: torch.Tensor, q_lat: torch.Tensor,
         kpos = pos.view(1, 1, -1)
         seen = (kpos <= qpos) & (qpos - kpos < window)
         s = s.masked_fill(~seen, float("-inf"))
-        p = torch.softmax(s, dim=-1)
-        out[:, start:start + qlen] = torch.einsum("hqn,nr->hqr", p, C
-                                                  ).to(out.dtype)
+        if sink is not None:
+            s = torch.cat([s, sink.float().view(H, 1, 1).expand(H, qlen, 1)],
+                          dim=-1)
+        p = torch.softmax(s, dim=-1)[..., :pos.numel()]
+        o = torch.einsum("hqn,nr->hqr", p, C)
+        if head_gate is not None:
+            o = o * torch.sigmoid(head_gate[start:start + qlen].float()
+                                  ).t().unsqueeze(-1)
+        out[:, start:start + qlen] = o.to(out.dtype)
 
 
 def sigmoid_gate_mul(out: torch.Tensor, a: torch.Tensor, g: torch.Tensor) -> None:
@@ -593,7 +602,7 @@ def short_conv_state(out: torch.Tensor, u: torch.Tensor, w: torch.Tensor,
         out[s0:s0 + n] = y.to(out.dtype)
 
 
-SCAN_GLA, SCAN_DELTA, SCAN_MLSTM = 0, 1, 2
+SCAN_GLA, SCAN_DELTA, SCAN_MLSTM, SCAN_DELTA_HEAD = 0, 1, 2, 3
 
 
 def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
@@ -613,7 +622,8 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
                 channel (gate [T, H*D]); S <- a S + k v^T; o = S^T q.
     SCAN_DELTA: g = exp(-exp(head_rate[h]) * softplus(gate + gate_bias)),
                 b = sigmoid(beta[t, h]); S <- g S; u = b (v - S^T k);
-                S <- S + k u^T; o = S^T q.
+                S <- S + k u^T; o = S^T q. gate [T, H*D].
+    SCAN_DELTA_HEAD: the same rule with one decay per head (gate [T, H]).
     SCAN_MLSTM: gate [T, 2H] = log-input | forget pre-activations,
                 i = c tanh((gate_i + bias_i) / c), f = logsigmoid(c tanh(
                 (gate_f + bias_f) / c)), c = gate_param; m' = max(f + m, i);
@@ -644,10 +654,10 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
                 a = torch.exp(lsig(z + gb) * gate_param).view(H, D)
                 St = St * a.unsqueeze(1) + vt.unsqueeze(2) * kt.unsqueeze(1)
                 out[t] = torch.einsum("hvd,hd->hv", St, qt)
-            elif kind == SCAN_DELTA:
+            elif kind in (SCAN_DELTA, SCAN_DELTA_HEAD):
                 g = torch.exp(-torch.exp(head_rate.float()).view(H, 1)
                               * torch.nn.functional.softplus(
-                                  (z + gb).view(H, D)))
+                                  (z + gb).view(H, -1)))
                 St = St * g.unsqueeze(1)
                 bt = torch.sigmoid(beta[t].float()).view(H, 1)
                 u = bt * (vt - torch.einsum("hvd,hd->hv", St, kt))
@@ -721,14 +731,15 @@ def routed_clamped_glu(out: torch.Tensor, gu: torch.Tensor,
     past n_experts belong to weightless experts and are ignored);
     g = min(gate, limit), u = clamp(up, -limit, limit);
     out[t, e, :] = weight[t, e] * g * sigmoid(slope * g) * (u + 1), and 0
-    where the weight is 0."""
+    where the weight is 0. weight None: every weight is 1."""
     T = gu.size(0)
     E = n_experts
     F_ = gu.size(1) // (2 * E)
     g3 = gu.view(T, E, 2 * F_).float()
     g = g3[..., :F_].clamp(max=limit)
     u = g3[..., F_:].clamp(-limit, limit)
-    w = weight[:, :E].float().unsqueeze(-1)
+    w = (torch.ones(T, E, 1) if weight is None
+         else weight[:, :E].float().unsqueeze(-1))
     y = g * torch.sigmoid(slope * g) * (u + 1.0) * w
     y = torch.where(w == 0, torch.zeros_like(y), y)
     out.copy_(y.view(T, E * F_).to(out.dtype))
@@ -774,12 +785,15 @@ def bigram_embed(x_out: torch.Tensor, ids: torch.Tensor, embed: torch.Tensor,
 
 
 def residual_update_norm(x_res: torch.Tensor, y, update: int, gate, gate_bias,
-                         rms_w, eps: float, norm_w, norm_b,
-                         h_out) -> None:
+                         rms_w, eps: float, norm_w, norm_b, h_out,
+                         rms_norm: bool = False, add_rows=None,
+                         add_vec=None) -> None:
     """fp32 residual update fused with the norm that feeds the next GEMM.
     update: NONE; SIGMOID_GATE x += sigmoid(gate + gate_bias) * y;
-    UNIT_RMS x += y / sqrt(mean(y^2) + eps) * rms_w. Then h_out = layer
-    norm of x ((x - mean) / sqrt(var + eps) * norm_w + norm_b), or just x
+    UNIT_RMS x += y / sqrt(mean(y^2) + eps) * rms_w. Then x += add_rows +
+    add_vec where given. Then h_out = layer
+    norm of x ((x - mean) / sqrt(var + eps) * norm_w + norm_b; rms_norm:
+    x / sqrt(mean(x^2) + eps) * norm_w + norm_b), or just x
     in h_out's dtype when norm_w is None; h_out None skips it."""
     if update == UPDATE_SIGMOID_GATE:
         g = gate.float()
@@ -788,17 +802,34 @@ def residual_update_norm(x_res: torch.Tensor, y, update: int, gate, gate_bias,
         x_res.add_(torch.sigmoid(g) * y.float())
     elif update == UPDATE_UNIT_RMS:
         x_res.add_(_unit(y.float(), eps) * rms_w.float())
+    if add_rows is not None:
+        x_res.add_(add_rows)
+    if add_vec is not None:
+        x_res.add_(add_vec)
     if h_out is None:
         return
     if norm_w is None:
         h_out.copy_(x_res.to(h_out.dtype))
         return
-    d = x_res - x_res.mean(-1, keepdim=True)
+    d = x_res if rms_norm else x_res - x_res.mean(-1, keepdim=True)
     r = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps)
     r = r * norm_w.float()
     if norm_b is not None:
         r = r + norm_b.float()
     h_out.copy_(r.to(h_out.dtype))
+
+
+def position_embed_norm(x_out: torch.Tensor, ids: torch.Tensor,
+                        positions: torch.Tensor, embed: torch.Tensor,
+                        pos: torch.Tensor, scale: float, w: torch.Tensor,
+                        eps: float, x_copy=None) -> None:
+    """x_out (fp32 [T, W]) = rms_norm(scale * embed[id] + pos[p]) * w, p the
+    token's position (clamped to the table); x_copy takes the same rows."""
+    p = positions.long().clamp(0, pos.size(0) - 1)
+    v = embed[ids].float() * scale + pos[p].float()
+    x_out.copy_(_unit(v, eps) * w.float())
+    if x_copy is not None:
+        x_copy.copy_(x_out)
 
 
 def xielu(out: torch.Tensor, z: torch.Tensor, coef: torch.Tensor) -> None:
