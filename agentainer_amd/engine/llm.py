@@ -1028,6 +1028,12 @@ class ModelInstance:
             want = [want[i] for i in live]
         if not entries:
             return torch.empty(0, self.cfg.vocab_size, device=self.device)
+        for seq_id, toks in entries:
+            n = self.kvm.seq_len(seq_id) + len(toks)
+            if n > self.cfg.max_position:
+                raise ValueError(f"sequence {seq_id!r} would hold {n} tokens; "
+                                 f"the model has {self.cfg.max_position} "
+                                 "positions")
         decode = all(len(t) == 1 and self.kvm.seq_len(s) > 0
                      for s, t in entries)
         if decode and len(entries) <= max(self.max_decode_batch, 1):

@@ -13,6 +13,7 @@ import torch
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
 import lelitar_oracle as O  # noqa: E402
+import mugazen_oracle as MO  # noqa: E402
 import pekarax_oracle as PO  # noqa: E402
 import sipelorn_oracle as SO  # noqa: E402
 import volalorn_oracle as VO  # noqa: E402
@@ -65,8 +66,25 @@ def _sipelorn_case():
     return _SipelornOracle, cfg, SO.random_weights(cfg, seed=24)
 
 
+class _MugazenOracle:
+    """The Mugazen oracle behind the other oracles' call signature."""
+    save_checkpoint = staticmethod(MO.save_checkpoint)
+
+    @staticmethod
+    def forward(cfg, w, tokens):
+        return MO.forward(tokens, w, cfg).float()
+
+
+def _mugazen_case():
+    cfg = MO.make_config(
+        [(MO.delta_layer(), MO.dense_mlp()), (MO.latent_layer(), MO.moe_mlp()),
+         (MO.delta_layer(), None)], vocab=120, loop=(1, 3, 2))
+    return _MugazenOracle, cfg, MO.random_weights(cfg, seed=25)
+
+
 @pytest.mark.parametrize("case", [_lelitar_case, _volalorn_case,
-                                  _pekarax_case, _sipelorn_case])
+                                  _pekarax_case, _sipelorn_case,
+                                  _mugazen_case])
 def test_trace_run_mixed_steps_match_oracle(tmp_path, case):
     O, cfg, w = case()
     model = str(tmp_path / "ckpt")
