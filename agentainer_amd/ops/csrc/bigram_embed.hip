@@ -98,7 +98,8 @@ __global__ void bigram_state_kernel(int* __restrict__ prev_state,
 
 constexpr int ROW_VALS = 32;   // values per thread: rows of up to 8192
 
-template <typename T, int NV>
+// NV groups of VEC consecutive values per thread hold the row
+template <typename T, int VEC, int NV>
 __global__ __launch_bounds__(256) void position_embed_kernel(
     float* __restrict__ x, float* __restrict__ x_copy,
     const long* __restrict__ ids, const int* __restrict__ positions,
@@ -112,22 +113,45 @@ __global__ __launch_bounds__(256) void position_embed_kernel(
   p = p < 0 ? 0 : (p >= n_pos ? n_pos - 1 : p);
   const T* er = embed + id * W;
   const T* pr = pos + (long)p * W;
-  float v[NV];
+  float v[NV][VEC];
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
-    const int i = k * 256 + threadIdx.x;
-    v[k] = i < W ? fmaf(ldf(er, i), scale, ldf(pr, i)) : 0.f;
-    ss = fmaf(v[k], v[k], ss);
+    const int i = (k * 256 + threadIdx.x) * VEC;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[k][j] = 0.f;
+    if (i < W) {
+      float p4[VEC];
+      if constexpr (VEC == 4) {
+        ld4(er, i, v[k]);
+        ld4(pr, i, p4);
+      } else {
+        v[k][0] = ldf(er, i);
+        p4[0] = ldf(pr, i);
+      }
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        v[k][j] = fmaf(v[k][j], scale, p4[j]);
+        ss = fmaf(v[k][j], v[k][j], ss);
+      }
+    }
   }
   const float rs = 1.0f / sqrtf(block_sum_256(ss, red) / (float)W + eps);
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
-    const int i = k * 256 + threadIdx.x;
+    const int i = (k * 256 + threadIdx.x) * VEC;
     if (i < W) {
-      const float o = v[k] * rs * w[i];
-      x[r * W + i] = o;
-      if (x_copy) x_copy[r * W + i] = o;
+      float wv[VEC];
+      if constexpr (VEC == 4) ld4(w, i, wv); else wv[0] = w[i];
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[k][j] *= rs * wv[j];
+      if constexpr (VEC == 4) {
+        st4(x, r * W + i, v[k]);
+        if (x_copy) st4(x_copy, r * W + i, v[k]);
+      } else {
+        x[r * W + i] = v[k][0];
+        if (x_copy) x_copy[r * W + i] = v[k][0];
+      }
     }
   }
 }
@@ -159,16 +183,21 @@ void position_embed_norm(torch::Tensor x, c10::optional<torch::Tensor> x_copy,
   }
   if (T_ == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-#define LAUNCH(N)                                                             \
-  hipLaunchKernelGGL((position_embed_kernel<T, N>), dim3(T_), dim3(256), 0,   \
+#define LAUNCH(V, N)                                                          \
+  hipLaunchKernelGGL((position_embed_kernel<T, V, N>), dim3(T_), dim3(256), 0,\
                      stream, x.data_ptr<float>(), xc, ids.data_ptr<long>(),   \
                      positions.data_ptr<int>(), (const T*)embed.data_ptr(),   \
                      (const T*)pos.data_ptr(), (float)scale,                  \
                      w.data_ptr<float>(), (float)eps, W, (long)embed.size(0), \
                      (int)pos.size(0))
   LATENT_DISPATCH_T(embed, {
-    if (W <= 256 * 8) LAUNCH(8);
-    else LAUNCH(ROW_VALS);
+    if (W % 4 == 0) {
+      if (W <= 256 * 4 * 2) LAUNCH(4, 2);
+      else if (W <= 256 * 4 * 4) LAUNCH(4, 4);
+      else LAUNCH(4, ROW_VALS / 4);
+    } else {
+      LAUNCH(1, ROW_VALS);
+    }
   });
 #undef LAUNCH
 }

@@ -331,6 +331,8 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
     const int groups = (W / 4 + 255) / 256;
     if (groups <= 2) {
       if (bf) LAUNCH(short, 4, 2); else LAUNCH(float, 4, 2);
+    } else if (groups <= 4) {
+      if (bf) LAUNCH(short, 4, 4); else LAUNCH(float, 4, 4);
     } else {
       if (bf) LAUNCH(short, 4, ROW_REGS); else LAUNCH(float, 4, ROW_REGS);
     }

@@ -121,6 +121,36 @@ __global__ __launch_bounds__(64) void grouped_route_kernel(
   }
 }
 
+__device__ __forceinline__ float clamped_unit(float g, float u, float limit,
+                                              float slope) {
+  const float gc = fminf(g, limit);
+  const float uc = fminf(fmaxf(u, -limit), limit);
+  return (gc / (1.0f + expf(-slope * gc))) * (uc + 1.0f);
+}
+
+// bf16, 8 values (16 bytes) per thread; one row of workgroups per token, so
+// no 64-bit division finds the place
+__global__ __launch_bounds__(256) void clamped_glu_bf16x8_kernel(
+    short* __restrict__ out, const short* __restrict__ gu,
+    const float* __restrict__ weight, long w_rs, int E, int F, long gu_rs,
+    float limit, float slope, int nbx) {
+  const unsigned t = blockIdx.x / (unsigned)nbx;
+  const int c = ((blockIdx.x % (unsigned)nbx) * 256 + threadIdx.x) * 8;
+  if (c >= E * F) return;
+  const int e = c / F, f = c - e * F;
+  const float w = weight ? weight[t * w_rs + e] : 1.0f;
+  bf16x8 o{};
+  if (w != 0.f) {
+    const short* p = gu + t * gu_rs + (long)e * 2 * F + f;
+    const bf16x8 g = *reinterpret_cast<const bf16x8*>(p);
+    const bf16x8 u = *reinterpret_cast<const bf16x8*>(p + F);
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      o[j] = f2bits(w * clamped_unit(bits2f(g[j]), bits2f(u[j]), limit, slope));
+  }
+  *reinterpret_cast<bf16x8*>(out + (long)t * E * F + c) = o;
+}
+
 template <typename T, int VEC>
 __global__ void clamped_glu_kernel(T* __restrict__ out,
                                    const T* __restrict__ gu,
@@ -148,11 +178,8 @@ __global__ void clamped_glu_kernel(T* __restrict__ out,
       u[0] = ldf(gu, base + F);
     }
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) {
-      const float gc = fminf(g[j], limit);
-      const float uc = fminf(fmaxf(u[j], -limit), limit);
-      o[j] = w * (gc / (1.0f + expf(-slope * gc))) * (uc + 1.0f);
-    }
+    for (int j = 0; j < VEC; ++j)
+      o[j] = w * clamped_unit(g[j], u[j], limit, slope);
   }
   if constexpr (VEC == 4) {
     st4(out, i, o);
@@ -214,6 +241,18 @@ void routed_clamped_glu(torch::Tensor out, torch::Tensor gu,
   const bool vec = F % 4 == 0 && gu.stride(0) % 4 == 0 &&
                    gu.storage_offset() % 4 == 0;
   auto stream = at::hip::getCurrentHIPStream();
+  const long nbx = ((long)E * F / 8 + 255) / 256;
+  if (out.scalar_type() == at::kBFloat16 && F % 8 == 0 &&
+      gu.stride(0) % 8 == 0 && nbx * T_ < (1L << 31) &&
+      reinterpret_cast<uintptr_t>(gu.data_ptr()) % 16 == 0 &&
+      reinterpret_cast<uintptr_t>(out.data_ptr()) % 16 == 0) {
+    hipLaunchKernelGGL(clamped_glu_bf16x8_kernel, dim3((unsigned)(nbx * T_)),
+                       dim3(256), 0, stream, (short*)out.data_ptr(),
+                       (const short*)gu.data_ptr(), wp, w_rs, E, F,
+                       (long)gu.stride(0), (float)limit, (float)slope,
+                       (int)nbx);
+    return;
+  }
   LATENT_DISPATCH_T(out, {
     if (vec) {
       hipLaunchKernelGGL((clamped_glu_kernel<T, 4>), dim3((n / 4 + 255) / 256),

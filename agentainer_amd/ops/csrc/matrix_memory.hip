@@ -135,6 +135,39 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
   }
 }
 
+// Four consecutive values per lane (8- or 16-byte accesses); LPR lanes cover
+// one head's row, 64 / LPR rows share a wave. Needs Dv <= 4 * LPR, Dv and the
+// gate's row stride multiples of 4.
+template <typename T, typename TG, int LPR>
+__global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(
+    T* __restrict__ out, const float* __restrict__ o,
+    const float* __restrict__ w, int w_shared, const TG* __restrict__ gate,
+    long gate_rs, float eps, bool silu_gate, long n_rows, int H, int Dv) {
+  const long row =
+      ((long)blockIdx.x * 4 + (threadIdx.x >> 6)) * (64 / LPR) +
+      (threadIdx.x & 63) / LPR;
+  const int i = (threadIdx.x % LPR) * 4;
+  const bool ok = row < n_rows && i < Dv;
+  float v[4] = {0.f, 0.f, 0.f, 0.f};
+  if (ok) ld4(o, row * Dv + i, v);
+  float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+#pragma unroll
+  for (int off = 1; off < LPR; off <<= 1) ss += __shfl_xor(ss, off, WAVE);
+  if (!ok) return;
+  const float r = 1.0f / sqrtf(ss / (float)Dv + eps);
+  const long t = row / H;
+  const int h = (int)(row - t * H);
+  float g[4], wv[4];
+  ld4(gate, t * gate_rs + (long)h * Dv + i, g);
+  ld4(w, (w_shared ? 0 : (long)h * Dv) + i, wv);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float sg = 1.0f / (1.0f + expf(-g[e]));
+    v[e] = v[e] * r * wv[e] * (silu_gate ? g[e] * sg : sg);
+  }
+  st4(out, row * Dv + i, v);
+}
+
 }  // namespace
 
 void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
@@ -293,8 +326,32 @@ void head_rmsnorm_gate(torch::Tensor out, torch::Tensor o, torch::Tensor w,
                      w.data_ptr<float>(), (int)(w.numel() == Dv),             \
                      (const TG*)gate.data_ptr(), (long)gate.stride(0),        \
                      (float)eps, silu_gate, n_rows, H, Dv)
+#define LAUNCH_VEC(TT, TG, L)                                                 \
+  hipLaunchKernelGGL((head_norm_gate_vec_kernel<TT, TG, L>),                  \
+                     dim3((n_rows + 4 * (64 / L) - 1) / (4 * (64 / L))),      \
+                     dim3(256), 0, stream, (TT*)out.data_ptr(),               \
+                     o.data_ptr<float>(), w.data_ptr<float>(),                \
+                     (int)(w.numel() == Dv), (const TG*)gate.data_ptr(),      \
+                     (long)gate.stride(0), (float)eps, silu_gate, n_rows, H,  \
+                     Dv)
+#define LAUNCH_VEC_L(TT, TG)                                                  \
+  do {                                                                        \
+    if (Dv <= 32) LAUNCH_VEC(TT, TG, 8);                                      \
+    else if (Dv <= 64) LAUNCH_VEC(TT, TG, 16);                                \
+    else if (Dv <= 128) LAUNCH_VEC(TT, TG, 32);                               \
+    else LAUNCH_VEC(TT, TG, 64);                                              \
+  } while (0)
+  const bool vec = Dv % 4 == 0 && Dv <= 256 && gate.stride(0) % 4 == 0 &&
+                   reinterpret_cast<uintptr_t>(gate.data_ptr()) %
+                           (4 * gate.element_size()) == 0;
   LATENT_DISPATCH_T(out, {
-    if (g_f32) LAUNCH(T, float); else LAUNCH(T, T);
+    if (vec) {
+      if (g_f32) LAUNCH_VEC_L(T, float); else LAUNCH_VEC_L(T, T);
+    } else {
+      if (g_f32) LAUNCH(T, float); else LAUNCH(T, T);
+    }
   });
 #undef LAUNCH
+#undef LAUNCH_VEC
+#undef LAUNCH_VEC_L
 }

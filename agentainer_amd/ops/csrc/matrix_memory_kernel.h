@@ -140,10 +140,10 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
 
   // ---- raw inputs of the next chunk, in registers. Wave w stages the
   // tokens c = w, w + WAVES, ... of a chunk for the whole workgroup; every
-  // lane keeps its own column's v; wave 0 evaluates the mLSTM gates, lane
-  // c those of token c.
+  // lane keeps its own column's v; wave 0 evaluates the mLSTM gates, the
+  // last wave the head-decay rule's two numbers, lane c those of token c.
   float rk[TPW][EPL], rq[TPW][EPL], rg[channel_decay(KIND) ? TPW : 1][EPL];
-  float rb[TPW], rz[KIND == KIND_DELTA_HEAD ? TPW : 1];
+  float rb[TPW];
   float rv[CH];
   float rgi = 0.f, rgf = 0.f;
   const TI* qp = (const TI*)a.q;
@@ -166,9 +166,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           if constexpr (channel_decay(KIND))
             rg[i][e] = ok ? a.gate[row * a.gate_rs + (long)h * D + rc] : 1.f;
         }
-        if constexpr (is_delta(KIND)) rb[i] = a.beta[row * a.beta_rs + h];
-        if constexpr (KIND == KIND_DELTA_HEAD)
-          rz[i] = a.gate[row * a.gate_rs + h];
+        if constexpr (KIND == KIND_DELTA) rb[i] = a.beta[row * a.beta_rs + h];
       }
     }
 #pragma unroll
@@ -180,6 +178,13 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         const long row = s0 + t0 + lane;
         rgi = a.gate[row * a.gate_rs + h];
         rgf = a.gate[row * a.gate_rs + H + h];
+      }
+    }
+    if constexpr (KIND == KIND_DELTA_HEAD) {
+      if (wave == WAVES - 1 && lane < CH && t0 + lane < n_tok) {
+        const long row = s0 + t0 + lane;
+        rgi = a.gate[row * a.gate_rs + h];
+        rgf = a.beta[row * a.beta_rs + h];
       }
     }
   };
@@ -219,11 +224,15 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         kq = wave_total(kq);
         if (lane == 0) {
           sc[c][0] = kq;
-          if constexpr (is_delta(KIND))
+          if constexpr (KIND == KIND_DELTA)
             sc[c][1] = 1.0f / (1.0f + expf(-rb[i]));
-          if constexpr (KIND == KIND_DELTA_HEAD)
-            sc[c][2] = expf(-rate * soft_plus(rz[i] + bias_i));
         }
+      }
+    }
+    if constexpr (KIND == KIND_DELTA_HEAD) {
+      if (wave == WAVES - 1 && lane < CH && t0 + lane < n_tok) {
+        sc[lane][1] = 1.0f / (1.0f + expf(-rgf));
+        sc[lane][2] = expf(-rate * soft_plus(rgi + bias_i));
       }
     }
     if constexpr (KIND == KIND_MLSTM) {
@@ -371,7 +380,14 @@ void launch_scan(const ScanArgs& a, int B, int lanes, hipStream_t stream) {
     ns = lanes < lo ? lo : (lanes > 16 ? 16 : lanes);
   } else {
     const long cols = (long)B * a.H * a.Dv;
-    while (ns < 16 && ns < lo * 4 && cols * ns / 64 < 4096) ns <<= 1;
+    if constexpr (KIND == KIND_DELTA_HEAD) {
+      // with no decay vectors to read, 16 rows per lane beat both 8 and 32
+      // from about a thousand waves on
+      ns = lo * 2 < 16 ? lo * 2 : 16;
+      while (ns < 16 && ns < lo * 4 && cols * ns / 64 < 1024) ns <<= 1;
+    } else {
+      while (ns < 16 && ns < lo * 4 && cols * ns / 64 < 4096) ns <<= 1;
+    }
   }
 #define SCAN_CASE(NS, RP)                                                     \
   hipLaunchKernelGGL((scan_kernel<KIND, TI, NS, RP>),                         \

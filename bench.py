@@ -86,7 +86,8 @@ def _parser():
                    help="--arch-compare: which size points to run "
                         "(default: all points of the design)")
     p.add_argument("--arch-design", default="lelitar",
-                   choices=["lelitar", "volalorn", "pekarax", "sipelorn"],
+                   choices=["lelitar", "volalorn", "pekarax", "sipelorn",
+                            "mugazen"],
                    help="--arch-compare: which design to measure")
     return p
 
@@ -300,6 +301,52 @@ def _sipelorn_points():
     }
 
 
+def _mugazen_points():
+    """Mugazen size points: four layer runs (a delta layer that runs twice,
+    then two latent-attention layers); the delta and the first latent layer
+    carry routed experts, the last a dense clamped unit of twice an expert's
+    size. 's' and 'l' stand beside the Sipelorn stacks of equal width, heads,
+    latent row, expert count, expert size and top-k (the closest existing
+    family: latent attention and SiLU experts), 's-pek' beside the Pekarax
+    stack (the closest recurrence), 's-mix' and 'l-mix' beside Mixtral."""
+    from agentainer_amd import ops
+    from agentainer_amd.models.lelitar import CAUSAL_WINDOW, LatentMixerConfig
+    from agentainer_amd.models.mugazen import (MugazenConfig,
+                                               MugazenFeedForwardConfig,
+                                               MugazenLayerConfig)
+    from agentainer_amd.models.pekarax import MatrixMemoryConfig
+
+    def mug(name, width, heads, ff, experts, top, q_rank, rank):
+        hv = width // 128
+        delta = MatrixMemoryConfig(ops.SCAN_DELTA_HEAD, hv, hv // 2, 128, 128,
+                                   conv_taps=4)
+        latent = LatentMixerConfig(
+            heads=heads, dim=128, vdim=128, q_rank=q_rank, kv_rank=rank,
+            window=CAUSAL_WINDOW, scale=128 ** -0.5, gate="head", sink=True)
+        moe = MugazenFeedForwardConfig("moe", ff, experts=experts, top=top)
+        dense = MugazenFeedForwardConfig("dense", 2 * ff, limit=7.0)
+        layers = [MugazenLayerConfig("delta", delta=delta, mlp=moe),
+                  MugazenLayerConfig("latent_attention", latent=latent,
+                                     mlp=moe),
+                  MugazenLayerConfig("latent_attention", latent=latent,
+                                     mlp=dense)]
+        return MugazenConfig(name=name, vocab_size=32000, hidden_size=width,
+                             layers=layers, norm_eps=1e-5, embed_scale=8.0,
+                             max_positions=4096, loop_start=0, loop_stop=1,
+                             loop_times=2)
+
+    s = mug("mugazen-s", 2048, 16, 4096, 8, 2, 768, 256)
+    lg = mug("mugazen-l", 4096, 32, 7168, 8, 2, 1536, 512)
+    sip, pek = _sipelorn_points(), _pekarax_points()
+    return {
+        "s": ("w2048-8x4096-top2", s, sip["s"][1], "sipelorn"),
+        "l": ("w4096-8x7168-top2", lg, sip["l"][1], "sipelorn"),
+        "s-pek": ("w2048-8x4096-top2", s, pek["s"][1], "pekarax"),
+        "s-mix": ("w2048-8x4096-top2", s, sip["s"][2], "mixtral"),
+        "l-mix": ("w4096-8x7168-top2", lg, sip["l"][2], "mixtral"),
+    }
+
+
 def run_arch_compare(args):
     """Prefill (8 x 1024-token prompts per step) and decode (64 sequences at
     1024 tokens of context, captured graph) throughput, through the
@@ -307,6 +354,7 @@ def run_arch_compare(args):
     from agentainer_amd.engine.llm import ModelInstance
     from agentainer_amd.models.lelitar import LelitarForCausalLM
     from agentainer_amd.models.mixtral import MixtralForCausalLM
+    from agentainer_amd.models.mugazen import MugazenForCausalLM
     from agentainer_amd.models.pekarax import PekaraxForCausalLM
     from agentainer_amd.models.sipelorn import SipelornForCausalLM
     from agentainer_amd.models.volalorn import VolalornForCausalLM
@@ -369,18 +417,21 @@ def run_arch_compare(args):
 
     design = args.arch_design
     pts = {"volalorn": _volalorn_points, "pekarax": _pekarax_points,
-           "sipelorn": _sipelorn_points, "lelitar": _arch_points}[design]()
+           "sipelorn": _sipelorn_points, "mugazen": _mugazen_points,
+           "lelitar": _arch_points}[design]()
+    cls_of = {"mixtral": MixtralForCausalLM, "pekarax": PekaraxForCausalLM,
+              "sipelorn": SipelornForCausalLM}
     ours_cls = {"volalorn": VolalornForCausalLM,
                 "pekarax": PekaraxForCausalLM,
                 "sipelorn": SipelornForCausalLM,
+                "mugazen": MugazenForCausalLM,
                 "lelitar": LelitarForCausalLM}[design]
     for key in (args.arch_sizes or ",".join(pts)).split(","):
         label, lcfg, rcfg, kind = pts[key.strip()]
         if small:  # CPU dry run: shrink to something that finishes
             continue
         ours = measure(lcfg.name, lcfg, ours_cls)
-        theirs = measure(rcfg.name, rcfg,
-                         MixtralForCausalLM if kind == "mixtral" else None)
+        theirs = measure(rcfg.name, rcfg, cls_of.get(kind))
         print(json.dumps({
             "metric": "arch_compare", "point": label, "layers": rcfg.n_layers,
             "prefill": f"{n_pf}x{pf_len}", "decode": f"{n_dec}@{ctx}",

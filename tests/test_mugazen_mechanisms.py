@@ -48,7 +48,7 @@ def i32(device, *vals):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("W", [40, 50, 2304])
+@pytest.mark.parametrize("W", [40, 50, 2304, 4352])
 def test_position_embedding_norm(device, dtype, W):
     V, P, scale, eps = 30, 17, 5.0, 1e-2
     embed, pos, nw = rnd(V, W, seed=1), rnd(P, W, seed=2, scale=2.0), rnd(
@@ -74,7 +74,7 @@ def test_position_embedding_norm(device, dtype, W):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("W", [64, 50, 1200, 4096])
+@pytest.mark.parametrize("W", [64, 50, 1200, 4096, 4100])
 def test_sandwich_residual_with_pass_inputs(device, dtype, W):
     """x += N(y; post); x += rows + vec; h = N(x; pre) — every optional
     part on and off; the mean of x is far from zero, so a layer norm in
