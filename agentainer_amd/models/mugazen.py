@@ -92,6 +92,17 @@ class LayerRun(NamedTuple):
     enters: bool              # first layer of its pass
 
 
+def layer_runs(n: int, start: int, stop: int, times: int) -> List[LayerRun]:
+    """Order in which n layers run when start .. stop-1 run `times` times in
+    a row (start == stop: no repeated group)."""
+    if stop <= start:
+        return [LayerRun(i, None, False) for i in range(n)]
+    return ([LayerRun(i, None, False) for i in range(start)]
+            + [LayerRun(i, t, i == start) for t in range(times)
+               for i in range(start, stop)]
+            + [LayerRun(i, None, False) for i in range(stop, n)])
+
+
 @dataclass
 class MugazenConfig:
     name: str = "tiny-mugazen"
@@ -120,13 +131,8 @@ class MugazenConfig:
         return self.loop_stop > self.loop_start
 
     def runs(self) -> List[LayerRun]:
-        a, b, n = self.loop_start, self.loop_stop, len(self.layers)
-        if not self.looped:
-            return [LayerRun(i, None, False) for i in range(n)]
-        return ([LayerRun(i, None, False) for i in range(a)]
-                + [LayerRun(i, t, i == a) for t in range(self.loop_times)
-                   for i in range(a, b)]
-                + [LayerRun(i, None, False) for i in range(b, n)])
+        return layer_runs(len(self.layers), self.loop_start, self.loop_stop,
+                          self.loop_times)
 
     def _kv_shapes(self):
         ls = [self.layers[r.layer] for r in self.runs()]

@@ -29,6 +29,10 @@ FAMILIES: Dict[str, Tuple[str, str, str, str]] = {
     # family's residual kernel
     "Mugazen": ("agentainer_amd.models.mugazen", "MUGAZEN_CONFIGS",
                 "make_mugazen_instance", "gated+latent+recurrent"),
+    # two attentions on the masked-attention kernels, the state-space scan,
+    # residual / embedding / narrow kernels of the gated module
+    "Larozen": ("agentainer_amd.models.larozen", "LAROZEN_CONFIGS",
+                "make_larozen_instance", "gated+masked+recurrent"),
 }
 
 

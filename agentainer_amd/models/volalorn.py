@@ -65,6 +65,10 @@ from .llama import AttnMetadata
 PROJ_ALIGN = 8
 
 
+def _align(n: int) -> int:
+    return -(-n // PROJ_ALIGN) * PROJ_ALIGN
+
+
 @dataclass
 class MaskedAttentionConfig:
     heads: int
@@ -95,8 +99,27 @@ class MaskedAttentionConfig:
     #                           taken off the score of key j at query p
     elem_gate: bool = False   # sigmoid gate per OUTPUT COORDINATE, read
     #                           from the mixer input
+    rot_pairs: bool = False   # the checkpoint rotates (2i, 2i+1) together;
+    #                           the serving order is (i, i + half)
+    rotate_only: bool = False  # rotary without any q/k norm
+    row_norm: bool = False    # weighted rms norm of q and of k over all
+    #                           heads of a token at once, no rotary
+    q_temp_coef: float = 0.0  # row_norm: q times 1 + coef *
+    q_temp_every: int = 1     # ln(floor((p + 1) / every) + 1) at position p
+    tied_values: bool = False  # the values are the keys as projected
+    sink: bool = False        # per-head score in the softmax denominator
+    out_bias: bool = False
     kv_from: Optional[int] = None   # this layer has no k/v projections: it
     #                           attends the pools of that (earlier) layer
+
+    @property
+    def pool_vdim(self) -> int:
+        """Coordinates of a value that the value pool keeps. A tied value
+        differs from its cached key only where the rotary turned it; from
+        there on the attention kernels read the key row."""
+        if not self.tied_values:
+            return self.vdim
+        return min(self.dim, max(_align(self.rot_dims), PROJ_ALIGN))
 
 
 @dataclass
@@ -198,10 +221,6 @@ def _param(*shape, dtype):
                               requires_grad=False)
 
 
-def _align(n: int) -> int:
-    return -(-n // PROJ_ALIGN) * PROJ_ALIGN
-
-
 class MaskedAttention(torch.nn.Module):
     """Grouped-query attention with a configurable mask, weighting, q/k
     normalization order and output gate (see MaskedAttentionConfig)."""
@@ -218,7 +237,8 @@ class MaskedAttention(torch.nn.Module):
         own_kv = mc.kv_from is None
         self.q_sz = H * mc.dim
         self.k_sz = G * mc.dim if own_kv else 0
-        self.v_sz = G * mc.vdim if own_kv else 0
+        # tied values have no rows of their own: they are the key columns
+        self.v_sz = G * mc.vdim if own_kv and not mc.tied_values else 0
         self.gate_sz = (H if mc.head_gate else
                         H * mc.vdim if mc.elem_gate else 0)
         # segment starts stay 16-byte aligned for the kernels' vector loads
@@ -232,6 +252,13 @@ class MaskedAttention(torch.nn.Module):
         f32 = torch.float32
         self.q_norm = _param(mc.dim, dtype=f32) if mc.norm_first else None
         self.k_norm = _param(mc.dim, dtype=f32) if mc.norm_first else None
+        if mc.row_norm:
+            self.q_norm = _param(self.q_sz, dtype=f32)
+            self.k_norm = _param(self.k_sz, dtype=f32)
+        self.norm_kind = (ops.NORM_OFF if mc.rotate_only else
+                          ops.NORM_FIRST if mc.norm_first else ops.NORM_LAST)
+        self.sink = _param(H, dtype=f32) if mc.sink else None
+        self.b_o = _param(width, dtype=dtype) if mc.out_bias else None
         self.key_bias = _param(H, dtype=f32) if mc.key_bias else None
         self.dist_bias = _param(H, 2, dtype=f32) if mc.dist_bias else None
         self.w_o = _param(width, H * mc.vdim, dtype=dtype)
@@ -242,18 +269,38 @@ class MaskedAttention(torch.nn.Module):
             mc.rot_dims, mc.rot_base, mc.rot_scaling)
         self.register_buffer("rot_freqs", freqs, persistent=False)
 
+    def _head_order(self, heads: int) -> Optional[torch.Tensor]:
+        """Row order that turns the checkpoint's neighbouring rotary pairs
+        (2i, 2i+1) of every head into the serving pairs (i, i + half); None
+        where nothing moves. Scores do not change under one permutation of q
+        and k; tied values are permuted with their keys, which the output
+        projection's columns undo."""
+        mc = self.mc
+        if not mc.rot_pairs or mc.rot_dims == 0:
+            return None
+        one = torch.tensor(list(range(0, mc.rot_dims, 2))
+                           + list(range(1, mc.rot_dims, 2))
+                           + list(range(mc.rot_dims, mc.dim)),
+                           dtype=torch.long, device=self.w_in.device)
+        at = torch.arange(heads, device=one.device) * mc.dim
+        return (at.unsqueeze(1) + one).reshape(-1)
+
     @torch.no_grad()
     def load(self, get, extra=None):
         """extra: weight rows [extra_rows, width] of the caller's
         projection."""
         mc = self.mc
+        q_order = self._head_order(mc.heads)
+        k_order = self._head_order(mc.kv_heads)
+        ordered = lambda t, o: t if o is None else t[o]     # noqa: E731
         own_kv = mc.kv_from is None
         q0, k0, v0 = 0, self.q_sz, self.q_sz + self.k_sz
         g0 = self.gate_off
         self.w_in.zero_()
-        self.w_in[q0:k0].copy_(get("q"))
+        self.w_in[q0:k0].copy_(ordered(get("q"), q_order))
         if own_kv:
-            self.w_in[k0:v0].copy_(get("k"))
+            self.w_in[k0:v0].copy_(ordered(get("k"), k_order))
+        if self.v_sz:
             self.w_in[v0:v0 + self.v_sz].copy_(get("v"))
         if self.gate_sz:
             self.w_in[g0:g0 + self.gate_sz].copy_(get("g"))
@@ -262,11 +309,12 @@ class MaskedAttention(torch.nn.Module):
                 extra)
         if mc.qkv_bias:
             self.b_in.zero_()
-            self.b_in[q0:k0].copy_(get("q.b"))
+            self.b_in[q0:k0].copy_(ordered(get("q.b"), q_order))
             if own_kv:
-                self.b_in[k0:v0].copy_(get("k.b"))
+                self.b_in[k0:v0].copy_(ordered(get("k.b"), k_order))
+            if self.v_sz:
                 self.b_in[v0:v0 + self.v_sz].copy_(get("v.b"))
-        if mc.norm_first:
+        if mc.norm_first or mc.row_norm:
             self.q_norm.copy_(get("q.norm").float())
             self.k_norm.copy_(get("k.norm").float())
         if mc.key_bias:
@@ -274,7 +322,14 @@ class MaskedAttention(torch.nn.Module):
         if mc.dist_bias:
             self.dist_bias.copy_(torch.stack(
                 [get("r1").float(), get("r2").float()], dim=1))
-        self.w_o.copy_(get("o"))
+        if mc.sink:
+            self.sink.copy_(get("sink").float())
+        w_o = get("o")
+        if mc.tied_values and q_order is not None:
+            w_o = w_o[:, q_order]
+        self.w_o.copy_(w_o)
+        if mc.out_bias:
+            self.b_o.copy_(get("o.b"))
         if mc.conv_taps > 0:
             # checkpoint [channels, taps] -> tap-major [taps, channels]
             names = ["q.conv"] + (["k.conv", "v.conv"] if own_kv else [])
@@ -296,7 +351,7 @@ class MaskedAttention(torch.nn.Module):
         manager's per-sequence state) is required when conv_taps > 0."""
         mc = self.mc
         cos_sin = None
-        if not mc.plain_qk:
+        if not (mc.plain_qk or mc.row_norm):
             key = self.rotary_key()
             cos_sin = tables.get(key) if tables is not None else None
             if cos_sin is None:
@@ -321,14 +376,23 @@ class MaskedAttention(torch.nn.Module):
         q = qkv[:, :k0].view(T, H, mc.dim)
         if own_kv:
             k = qkv[:, k0:v0].view(T, G, mc.dim)
-            v = qkv[:, v0:c_end].view(T, G, mc.vdim)
-            if mc.plain_qk:
+            if mc.tied_values:
+                v = k[:, :, :mc.pool_vdim]
+            else:
+                v = qkv[:, v0:c_end].view(T, G, mc.vdim)
+            if mc.row_norm:
+                ops.row_norm_append(qkv[:, :k0], qkv[:, k0:v0],
+                                    qkv[:, v0:c_end], k_cache, v_cache,
+                                    md.positions, md.slot_mapping, self.eps,
+                                    self.q_norm, self.k_norm, mc.q_temp_coef,
+                                    mc.q_temp_every)
+            elif mc.plain_qk:
                 ops.head_kv_append(k, v, k_cache, v_cache,
                                    md.slot_mapping)
             else:
                 ops.rotary_norm_append(q, k, v, k_cache, v_cache, cos_sin,
                                        md.slot_mapping, self.eps, self.q_norm,
-                                       self.k_norm, mc.norm_first)
+                                       self.k_norm, self.norm_kind)
         out = torch.empty(T, H, mc.vdim, dtype=h.dtype, device=h.device)
         ops.masked_attention(
             out, q, k_cache, v_cache, md.page_table, md.seq_lens,
@@ -338,8 +402,8 @@ class MaskedAttention(torch.nn.Module):
             mc.sigmoid_weights, mc.softcap, self.key_bias,
             proj[:, g0:g0 + self.gate_sz] if self.gate_sz else None,
             max_qlen=md.max_qlen if md.is_prefill else 1,
-            dist_bias=self.dist_bias)
-        y = ops.linear(out.view(T, H * mc.vdim), self.w_o)
+            dist_bias=self.dist_bias, sink=self.sink)
+        y = ops.linear(out.view(T, H * mc.vdim), self.w_o, bias=self.b_o)
         if self.extra_rows:
             return y, proj[:, self.extra_off:self.extra_off + self.extra_rows]
         return y

@@ -250,6 +250,16 @@ def linear(x: torch.Tensor, w: torch.Tensor,
     return torch.nn.functional.linear(x, w, bias)
 
 
+def linear_fp32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x[M,K] @ w[N,K]^T in the operands' precision with an fp32 result that
+    is never rounded to bf16: for products that ARE the residual stream."""
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, w)
+    if x.is_cuda:
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return torch.nn.functional.linear(x.float(), w.float())
+
+
 def quantize_weight_fp8(w: torch.Tensor):
     """Offline per-output-channel OCP e4m3 quantization of a [N, K] weight:
     returns (fragment-linear packed bytes, f32 scales[N]). Serves the fp8
@@ -531,8 +541,8 @@ def routed_scaled_silu_mul(out, gu, weight):
 
 # ---------------------------------------------------------------------
 # Scalar-gain post-norm, PolyNorm, partial rotary (+YaRN) with q/k norms,
-# masked attention (chunk / window masks; softmax or sigmoid weights) over
-# per-head K/V pools. Own extension (_hip_masked.so), same policy: required
+# row-wide q/k norms with a query temperature, masked attention (chunk /
+# window masks; softmax or sigmoid weights; sinks) over per-head K/V pools. Own extension (_hip_masked.so), same policy: required
 # on a GPU, fp32 torch references on CPU.
 # ---------------------------------------------------------------------
 
@@ -581,6 +591,9 @@ MASK_CAUSAL = reference.MASK_CAUSAL
 MASK_WINDOW = reference.MASK_WINDOW
 MASK_CHUNK = reference.MASK_CHUNK
 rotary_frequencies = reference.rotary_frequencies
+NORM_LAST = reference.NORM_LAST
+NORM_FIRST = reference.NORM_FIRST
+NORM_OFF = reference.NORM_OFF
 
 
 def scalar_postnorm_residual(x_res, y, gain, eps: float, h_out):
@@ -621,15 +634,33 @@ def rotary_table(positions, freqs, amp: float):
 
 def rotary_norm_append(q, k, v, k_cache, v_cache, cos_sin, slot_mapping,
                        eps: float, q_w=None, k_w=None,
-                       norm_first: bool = False):
+                       norm: int = NORM_LAST):
+    """norm: unit rms after the rotation, weighted rms norm before it
+    (q_w / k_w), or no norm (see reference.rotary_norm_append)."""
     mod = _dispatch_masked("rotary_norm_append", q)
     if mod:
         mod.rotary_norm_append(q, k, v, k_cache, v_cache, cos_sin,
                                slot_mapping, float(eps), q_w, k_w,
-                               bool(norm_first))
+                               int(norm))
     else:
         reference.rotary_norm_append(q, k, v, k_cache, v_cache, cos_sin,
-                                     slot_mapping, eps, q_w, k_w, norm_first)
+                                     slot_mapping, eps, q_w, k_w, norm)
+
+
+def row_norm_append(q, k, v, k_cache, v_cache, positions, slot_mapping,
+                    eps: float, q_w, k_w, temp_coef: float = 0.0,
+                    temp_every: int = 1):
+    """RMS norm of q [T, H*D] (in place) and k [T, G*D] over whole rows,
+    query temperature, K/V append (see reference.row_norm_append)."""
+    mod = _dispatch_masked("row_norm_append", q)
+    if mod:
+        mod.row_norm_append(q, k, v, k_cache, v_cache, positions,
+                            slot_mapping, float(eps), q_w, k_w,
+                            float(temp_coef), int(temp_every))
+    else:
+        reference.row_norm_append(q, k, v, k_cache, v_cache, positions,
+                                  slot_mapping, eps, q_w, k_w, temp_coef,
+                                  temp_every)
 
 
 # AGENTAINER_MASKED_SIMPLE=1 forces the one-wave-per-row kernel (A/B and
@@ -644,9 +675,11 @@ def masked_attention(out, q, k_cache, v_cache, page_table, seq_lens,
                      mask_size: int, keep_first: int = 0,
                      sigmoid_weights: bool = False, softcap: float = 0.0,
                      key_bias=None, head_gate=None, max_qlen: int = 1,
-                     dist_bias=None):
+                     dist_bias=None, sink=None):
     """dist_bias: fp32 [H, 2] = (r1, r2) per head; r1 * ln(1 + r2 * distance)
-    is taken off every score (see reference.masked_attention)."""
+    is taken off every score; sink: fp32 [H], exp(sink_h) joins head h's
+    softmax denominator; v_cache may hold only the leading coordinates of
+    values that end like their keys (see reference.masked_attention)."""
     mod = _dispatch_masked("masked_attention", q)
     if mod:
         mod.masked_attention(out, q, k_cache, v_cache, page_table, seq_lens,
@@ -654,21 +687,21 @@ def masked_attention(out, q, k_cache, v_cache, page_table, seq_lens,
                              int(mask_kind), int(mask_size), int(keep_first),
                              bool(sigmoid_weights), float(softcap), key_bias,
                              head_gate, int(max_qlen), bool(MASKED_SIMPLE),
-                             int(MASKED_SPLITS), dist_bias)
+                             int(MASKED_SPLITS), dist_bias, sink)
     else:
         reference.masked_attention(out, q, k_cache, v_cache, page_table,
                                    seq_lens, query_starts, query_lens, scale,
                                    mask_kind, mask_size, keep_first,
                                    sigmoid_weights, softcap, key_bias,
-                                   head_gate, dist_bias)
+                                   head_gate, dist_bias, sink)
     return out
 
 
 # ---------------------------------------------------------------------
 # Post-norm residual with (1 + w) RMS norm, short causal convolutions with
 # a per-sequence tail, matrix-memory recurrences (gated linear attention,
-# gated delta rules, mLSTM) over per-sequence state, per-head output norm +
-# gate, group-limited softmax routing and clamped gated experts. Own
+# gated delta rules, mLSTM, state-space) over per-sequence state, per-head
+# output norm + gate, gate + grouped norm, group-limited softmax routing and clamped gated experts. Own
 # extension (_hip_recurrent.so), same policy: required on a GPU, fp32
 # torch references on CPU.
 # ---------------------------------------------------------------------
@@ -718,6 +751,7 @@ SCAN_GLA = reference.SCAN_GLA
 SCAN_DELTA = reference.SCAN_DELTA
 SCAN_MLSTM = reference.SCAN_MLSTM
 SCAN_DELTA_HEAD = reference.SCAN_DELTA_HEAD
+SCAN_SSD = reference.SCAN_SSD
 
 
 def postln_rmsnorm_residual(x_res, y, w1p, eps: float, h_out,
@@ -739,19 +773,19 @@ def postln_rmsnorm_residual(x_res, y, w1p, eps: float, h_out,
 def short_conv_state(out, u, w, tail, state_slots, seq_lens, query_starts,
                      query_lens, silu: bool = False, norm_channels: int = 0,
                      head_dim: int = 1, lead_channels: int = 0,
-                     lead_scale: float = 1.0, l2_eps: float = 1e-6):
+                     lead_scale: float = 1.0, l2_eps: float = 1e-6, bias=None):
     mod = _dispatch_recurrent("short_conv_state", u)
     if mod:
         mod.short_conv_state(out, u, w, tail, state_slots, seq_lens,
                              query_starts, query_lens, bool(silu),
                              int(norm_channels), int(head_dim),
                              int(lead_channels), float(lead_scale),
-                             float(l2_eps))
+                             float(l2_eps), bias)
     else:
         reference.short_conv_state(out, u, w, tail, state_slots, seq_lens,
                                    query_starts, query_lens, silu,
                                    norm_channels, head_dim, lead_channels,
-                                   lead_scale, l2_eps)
+                                   lead_scale, l2_eps, bias)
     return out
 
 
@@ -763,19 +797,29 @@ SCAN_LANES = int(os.environ.get("AGENTAINER_SCAN_LANES", "0"))
 def matrix_memory_scan(kind: int, out, q, k, v, gate, gate_bias, head_rate,
                        beta, q_scale: float, gate_param: float, S, n_state,
                        m_state, state_slots, seq_lens, query_starts,
-                       query_lens):
+                       query_lens, skip=None):
     mod = _dispatch_recurrent("matrix_memory_scan", q)
     if mod:
         mod.matrix_memory_scan(int(kind), out, q, k, v, gate, gate_bias,
                                head_rate, beta, float(q_scale),
                                float(gate_param), S, n_state, m_state,
                                state_slots, seq_lens, query_starts,
-                               query_lens, int(SCAN_LANES))
+                               query_lens, int(SCAN_LANES), skip)
     else:
         reference.matrix_memory_scan(kind, out, q, k, v, gate, gate_bias,
                                      head_rate, beta, q_scale, gate_param, S,
                                      n_state, m_state, state_slots, seq_lens,
-                                     query_starts, query_lens)
+                                     query_starts, query_lens, skip)
+    return out
+
+
+def gate_group_rmsnorm(out, o, w, z, parts: int, eps: float):
+    """out = (o * silu(z)) RMS-normed in `parts` equal parts, times w."""
+    mod = _dispatch_recurrent("gate_group_rmsnorm", o)
+    if mod:
+        mod.gate_group_rmsnorm(out, o, w, z, int(parts), float(eps))
+    else:
+        reference.gate_group_rmsnorm(out, o, w, z, parts, eps)
     return out
 
 
@@ -814,8 +858,8 @@ def routed_clamped_glu(out, gu, weight, n_experts: int, limit: float,
 
 
 # ---------------------------------------------------------------------
-# Hashed bigram embedding, learned-position embedding, sigmoid-gated or
-# unit-rms residual + layer or RMS norm, xIELU,
+# Plain, hashed bigram and learned-position embeddings, sigmoid-gated,
+# unit-rms or plain residual + layer or RMS norm, xIELU, squared ReLU,
 # token-side gate, sigmoid group-limited routing, output-weighted gated
 # experts with a tail expert, latent rotary append, plain K/V append and
 # an elementwise output gate. Own extension (_hip_gated.so), same policy:
@@ -866,6 +910,7 @@ def _dispatch_gated(name: str, t: torch.Tensor):
 UPDATE_NONE = reference.UPDATE_NONE
 UPDATE_SIGMOID_GATE = reference.UPDATE_SIGMOID_GATE
 UPDATE_UNIT_RMS = reference.UPDATE_UNIT_RMS
+UPDATE_ADD = reference.UPDATE_ADD
 
 
 def bigram_embed(x_out, ids, embed, bigram, scale: float, mul_prev: int,
@@ -887,20 +932,34 @@ def bigram_embed(x_out, ids, embed, bigram, scale: float, mul_prev: int,
 def residual_update_norm(x_res, y, update: int, gate, gate_bias, rms_w,
                          eps: float, norm_w, norm_b, h_out,
                          rms_norm: bool = False, add_rows=None,
-                         add_vec=None):
+                         add_vec=None, y2=None, rms_w2=None):
     """rms_norm: h_out is the RMS norm of the stream instead of the layer
     norm; add_rows [T, W] / add_vec [W] (fp32) join the stream after the
-    update and before the norm (see reference.residual_update_norm)."""
+    update and before the norm; y2 / rms_w2: a second output of a unit-rms
+    update (see reference.residual_update_norm). h_out may be a column range
+    of a wider matrix."""
     mod = _dispatch_gated("residual_update_norm", x_res)
     if mod:
         mod.residual_update_norm(x_res, y, int(update), gate, gate_bias,
                                  rms_w, float(eps), norm_w, norm_b,
-                                 bool(rms_norm), add_rows, add_vec, h_out)
+                                 bool(rms_norm), add_rows, add_vec, h_out, y2,
+                                 rms_w2)
     else:
         reference.residual_update_norm(x_res, y, update, gate, gate_bias,
                                        rms_w, eps, norm_w, norm_b, h_out,
-                                       rms_norm, add_rows, add_vec)
+                                       rms_norm, add_rows, add_vec, y2,
+                                       rms_w2)
     return h_out
+
+
+def embed_rows(ids, embed, x_out=None, raw=None):
+    """x_out (fp32) and / or raw (the table's type, may be a column range of
+    a wider matrix) = embed[ids]."""
+    mod = _dispatch_gated("embed_rows", ids)
+    if mod:
+        mod.embed_rows(x_out, raw, ids, embed)
+    else:
+        reference.embed_rows(ids, embed, x_out, raw)
 
 
 def position_embed_norm(x_out, ids, positions, embed, pos, scale: float, w,
@@ -937,6 +996,15 @@ def xielu(out, z, coef):
         mod.xielu(out, z, coef)
     else:
         reference.xielu(out, z, coef)
+    return out
+
+
+def relu_square(out, z):
+    mod = _dispatch_gated("relu_square", z)
+    if mod:
+        mod.relu_square(out, z)
+    else:
+        reference.relu_square(out, z)
     return out
 
 

@@ -40,11 +40,13 @@ LATENT_SOURCES = [
     "routed_ffn.hip",
 ]
 
-# scalar-gain norms, PolyNorm, rotary + q/k norm + append, masked attention
+# scalar-gain norms, PolyNorm, rotary + q/k norm + append, row-wide q/k norm +
+# append, masked attention
 MASKED_SOURCES = [
     "masked_bindings.cpp",
     "scalar_norm.hip",
     "rotary_norm.hip",
+    "row_norm.hip",
     "masked_attn.hip",
 ]
 
@@ -58,6 +60,7 @@ RECURRENT_SOURCES = [
     "matrix_memory_gla.hip",
     "matrix_memory_delta.hip",
     "matrix_memory_mlstm.hip",
+    "matrix_memory_ssd.hip",
     "grouped_route.hip",
 ]
 

@@ -1,4 +1,10 @@
-// Token embeddings with a second table (gfx950).
+// Token embeddings (gfx950).
+//
+// embed_rows: the table's rows as the fp32 stream, and as they are into a
+// column range of a wider matrix (the input of a projection that reads the
+// embedding again).
+//
+// With a second table:
 //
 // position_embed_norm: x[r] = rms_norm(scale * embed[id_r] + pos[p_r]) * w,
 // fp32 out, optionally written twice (the second copy is what later passes
@@ -83,6 +89,28 @@ __global__ __launch_bounds__(256) void bigram_embed_kernel(
   }
 }
 
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void embed_rows_kernel(
+    float* __restrict__ x, T* __restrict__ raw, long raw_rs,
+    const long* __restrict__ ids, const T* __restrict__ embed, int W,
+    long vocab) {
+  const long r = blockIdx.x;
+  long id = ids[r];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  for (int i = threadIdx.x * VEC; i < W; i += 256 * VEC) {
+    float v[VEC];
+    if constexpr (VEC == 4) {
+      ld4(embed, id * W + i, v);
+      if (x) st4(x, r * W + i, v);
+      if (raw) st4(raw, r * raw_rs + i, v);
+    } else {
+      v[0] = ldf(embed, id * W + i);
+      if (x) x[r * W + i] = v[0];
+      if (raw) stf(raw, r * raw_rs + i, v[0]);
+    }
+  }
+}
+
 __global__ void bigram_state_kernel(int* __restrict__ prev_state,
                                     const long* __restrict__ ids,
                                     const long* __restrict__ slots,
@@ -157,6 +185,41 @@ __global__ __launch_bounds__(256) void position_embed_kernel(
 }
 
 }  // namespace
+
+void embed_rows(c10::optional<torch::Tensor> x,
+                c10::optional<torch::Tensor> raw, torch::Tensor ids,
+                torch::Tensor embed) {
+  TORCH_CHECK(ids.scalar_type() == at::kLong && ids.is_contiguous());
+  TORCH_CHECK(embed.dim() == 2 && embed.is_contiguous() && embed.size(0) >= 1);
+  const int T_ = ids.numel(), W = embed.size(1);
+  float* xp = nullptr;
+  void* rp = nullptr;
+  long raw_rs = 0;
+  bool vec = W % 4 == 0;
+  if (x.has_value()) {
+    TORCH_CHECK(x->scalar_type() == at::kFloat && x->is_contiguous() &&
+                x->dim() == 2 && x->size(0) == T_ && x->size(1) == W);
+    xp = x->data_ptr<float>();
+  }
+  if (raw.has_value()) {
+    TORCH_CHECK(raw->scalar_type() == embed.scalar_type() && raw->dim() == 2 &&
+                raw->size(0) == T_ && raw->size(1) == W &&
+                raw->stride(1) == 1);
+    rp = raw->data_ptr();
+    raw_rs = raw->stride(0);
+    vec = vec && raw_rs % 4 == 0 && raw->storage_offset() % 4 == 0;
+  }
+  if (T_ == 0 || (!xp && !rp)) return;
+  auto stream = at::hip::getCurrentHIPStream();
+#define LAUNCH(V)                                                             \
+  hipLaunchKernelGGL((embed_rows_kernel<T, V>), dim3(T_), dim3(256), 0,       \
+                     stream, xp, (T*)rp, raw_rs, ids.data_ptr<long>(),        \
+                     (const T*)embed.data_ptr(), W, (long)embed.size(0))
+  LATENT_DISPATCH_T(embed, {
+    if (vec) LAUNCH(4); else LAUNCH(1);
+  });
+#undef LAUNCH
+}
 
 void position_embed_norm(torch::Tensor x, c10::optional<torch::Tensor> x_copy,
                          torch::Tensor ids, torch::Tensor positions,

@@ -1,6 +1,6 @@
 // pybind11 bindings: hashed bigram embedding, learned-position embedding,
-// gated residual + layer or RMS norm, xIELU, token-side gate, sigmoid group-limited routing, output-weighted
-// gated experts, latent rotary append, plain K/V append, output gate,
+// gated residual + layer or RMS norm, xIELU, squared ReLU, token-side gate,
+// sigmoid group-limited routing, output-weighted gated experts, latent rotary append, plain K/V append, output gate,
 // narrow projections with an fp32 result.
 #include <torch/extension.h>
 
@@ -13,7 +13,9 @@ void bigram_embed(torch::Tensor x, torch::Tensor ids, torch::Tensor embed,
 void residual_update_norm(torch::Tensor x, OptT y, long update, OptT gate,
                           OptT gate_bias, OptT rms_w, double eps, OptT norm_w,
                           OptT norm_b, bool rms_norm, OptT add_rows,
-                          OptT add_vec, OptT h);
+                          OptT add_vec, OptT h, OptT y2, OptT rms_w2);
+void relu_square(torch::Tensor out, torch::Tensor z);
+void embed_rows(OptT x, OptT raw, torch::Tensor ids, torch::Tensor embed);
 void position_embed_norm(torch::Tensor x, OptT x_copy, torch::Tensor ids,
                          torch::Tensor positions, torch::Tensor embed,
                          torch::Tensor pos, double scale, torch::Tensor w,
@@ -42,7 +44,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("bigram_embed", &bigram_embed,
         "scaled embedding + hashed bigram row; previous token kept as state");
   m.def("residual_update_norm", &residual_update_norm,
-        "gated / unit-rms fp32 residual update fused with a layer / RMS norm");
+        "gated / unit-rms / plain fp32 residual update fused with a layer / RMS "
+        "norm");
+  m.def("relu_square", &relu_square, "max(z, 0)^2");
+  m.def("embed_rows", &embed_rows,
+        "embedding rows as the fp32 stream and / or as they are");
   m.def("position_embed_norm", &position_embed_norm,
         "RMS norm of scale * embedding + learned position row");
   m.def("narrow_linear", &narrow_linear,

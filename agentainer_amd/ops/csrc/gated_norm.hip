@@ -5,18 +5,22 @@
 //                            nothing
 //                            x += sigmoid(gate + gate_bias) * y
 //                            x += y / sqrt(mean(y^2) + eps) * rms_w
+//                              (+ the same of a second y2, rms_w2)
+//                            x += y
 //                          then optionally x += add_rows[row] + add_vec (what
 //                          a repeated group of layers takes in before a pass),
 //                          and then h = ((x - mean) / sqrt(var + eps)) * w + b
 //                          or, as an RMS norm, h = x / sqrt(mean(x^2) + eps) *
 //                          w + b in the compute dtype (the next GEMM's input),
-//                          or h = x cast (no norm weights), or nothing.
+//                          or h = x cast (no norm weights), or nothing. h may
+//                          be a column range of a wider matrix.
 //                          One 256-thread workgroup per row; the updated row
 //                          stays in registers between the passes (rows up to
 //                          256 * 4 * ROW_REGS values), so x is read and
 //                          written once. The variance is the mean of squared
 //                          deviations (second pass over registers), not
 //                          E[x^2] - mean^2.
+//   relu_square            max(z, 0)^2
 //   xielu                  z > 0: a_p z^2 + z/2; z <= 0: a_n (e^z - 1 - z) + z/2
 //   gelu_gate_rows         out[r, d] = gelu_tanh(t[r, d]) * table[ids[r], c0 + d]
 //   sigmoid_gate_rows      out[r, c] = a[r, c] * sigmoid(gate[r, c])
@@ -29,7 +33,7 @@
 
 namespace {
 
-constexpr int UPD_NONE = 0, UPD_GATE = 1, UPD_RMS = 2;
+constexpr int UPD_NONE = 0, UPD_GATE = 1, UPD_RMS = 2, UPD_ADD = 3;
 constexpr int ROW_REGS = 8;   // float4 groups per thread: rows <= 8192 values
 
 template <typename T, int VEC>
@@ -58,19 +62,18 @@ template <typename T, int VEC, int NREG>
 __global__ __launch_bounds__(256) void residual_update_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, long y_rs, int update,
     const T* __restrict__ gate, long g_rs, const float* __restrict__ gate_bias,
-    const float* __restrict__ rms_w, float eps,
+    const float* __restrict__ rms_w, const T* __restrict__ y2, long y2_rs,
+    const float* __restrict__ rms_w2, float eps,
     const float* __restrict__ norm_w, const float* __restrict__ norm_b,
     bool rms_norm, const float* __restrict__ add_rows,
-    const float* __restrict__ add_vec, T* __restrict__ h, int W) {
+    const float* __restrict__ add_vec, T* __restrict__ h, long h_rs, int W) {
   __shared__ float red[4];
   const long row = blockIdx.x;
   float* xr = x + row * W;
   const float inv_w = 1.0f / (float)W;
   float xv[NREG][VEC];
 
-  float scale_y = 1.0f;
-  if (update == UPD_RMS) {
-    const T* yr = y + row * y_rs;
+  auto unit_scale = [&](const T* yr) {
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < NREG; ++k) {
@@ -82,7 +85,12 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
         for (int j = 0; j < VEC; ++j) ss = fmaf(v[j], v[j], ss);
       }
     }
-    scale_y = 1.0f / sqrtf(block_sum_256(ss, red) * inv_w + eps);
+    return 1.0f / sqrtf(block_sum_256(ss, red) * inv_w + eps);
+  };
+  float scale_y = 1.0f, scale_y2 = 0.f;
+  if (update == UPD_RMS) {
+    scale_y = unit_scale(y + row * y_rs);
+    if (y2) scale_y2 = unit_scale(y2 + row * y2_rs);
   }
 
   float sum = 0.f;
@@ -110,6 +118,18 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
 #pragma unroll
         for (int j = 0; j < VEC; ++j)
           xv[k][j] = fmaf(v[j] * scale_y, w[j], xv[k][j]);
+        if (y2) {
+          ldv<T, VEC>(y2 + row * y2_rs, i, v);
+          ldv<float, VEC>(rms_w2, i, w);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j)
+            xv[k][j] = fmaf(v[j] * scale_y2, w[j], xv[k][j]);
+        }
+      } else if (update == UPD_ADD) {
+        float v[VEC];
+        ldv<T, VEC>(y + row * y_rs, i, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) xv[k][j] += v[j];
       }
       if (add_rows) {
         float v[VEC];
@@ -130,7 +150,7 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
     }
   }
   if (h == nullptr) return;
-  T* hr = h + row * W;
+  T* hr = h + row * h_rs;
   if (norm_w == nullptr) {
 #pragma unroll
     for (int k = 0; k < NREG; ++k) {
@@ -166,6 +186,35 @@ __global__ __launch_bounds__(256) void residual_update_norm_kernel(
       for (int j = 0; j < VEC; ++j) o[j] = fmaf(xv[k][j] * r, w[j], b[j]);
       stv<T, VEC>(hr, i, o);
     }
+  }
+}
+
+template <typename T, int VEC>
+__global__ void relu_square_kernel(T* __restrict__ out,
+                                   const T* __restrict__ z, long z_rs, long n,
+                                   int C) {
+  const long i = ((long)blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+  if (i >= n) return;
+  const long r = i / C;
+  const int c = (int)(i - r * C);
+  if constexpr (VEC == 8) {
+    const bf16x8 v = *reinterpret_cast<const bf16x8*>(z + r * z_rs + c);
+    bf16x8 o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float a = fmaxf(bits2f(v[j]), 0.f);
+      o[j] = f2bits(a * a);
+    }
+    *reinterpret_cast<bf16x8*>(out + i) = o;
+  } else {
+    float v[VEC];
+    ldv<T, VEC>(z, r * z_rs + c, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float a = fmaxf(v[j], 0.f);
+      v[j] = a * a;
+    }
+    stv<T, VEC>(out, i, v);
   }
 }
 
@@ -258,11 +307,13 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
                           c10::optional<torch::Tensor> norm_b, bool rms_norm,
                           c10::optional<torch::Tensor> add_rows,
                           c10::optional<torch::Tensor> add_vec,
-                          c10::optional<torch::Tensor> h) {
+                          c10::optional<torch::Tensor> h,
+                          c10::optional<torch::Tensor> y2,
+                          c10::optional<torch::Tensor> rms_w2) {
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.is_contiguous() &&
               x.dim() == 2);
   const int rows = x.size(0), W = x.size(1);
-  TORCH_CHECK(update >= UPD_NONE && update <= UPD_RMS);
+  TORCH_CHECK(update >= UPD_NONE && update <= UPD_ADD);
   TORCH_CHECK(W <= 256 * 4 * ROW_REGS, "row wider than ", 256 * 4 * ROW_REGS);
   auto check_vec = [&](const c10::optional<torch::Tensor>& t) {
     if (t.has_value())
@@ -271,6 +322,7 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
   };
   check_vec(gate_bias);
   check_vec(rms_w);
+  check_vec(rms_w2);
   check_vec(norm_w);
   check_vec(norm_b);
   check_vec(add_vec);
@@ -279,14 +331,14 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
                 add_rows->is_contiguous() && add_rows->dim() == 2 &&
                 add_rows->size(0) == rows && add_rows->size(1) == W);
   bool vec = W % 4 == 0;
-  long y_rs = 0, g_rs = 0;
+  long y_rs = 0, y2_rs = 0, g_rs = 0, h_rs = 0;
   at::ScalarType ct = at::kFloat;
   bool have_ct = false;
   auto check_rows = [&](const torch::Tensor& t) {
     TORCH_CHECK(t.dim() == 2 && t.size(0) == rows && t.size(1) == W &&
                 t.stride(1) == 1);
     TORCH_CHECK(!have_ct || t.scalar_type() == ct,
-                "y, gate and h share one element type");
+                "y, y2, gate and h share one element type");
     ct = t.scalar_type();
     have_ct = true;
     vec = vec && aligned_rows(t, 4);
@@ -302,9 +354,17 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
     g_rs = gate->stride(0);
   }
   if (update == UPD_RMS) TORCH_CHECK(rms_w.has_value());
+  TORCH_CHECK(y2.has_value() == rms_w2.has_value() &&
+              (!y2.has_value() || update == UPD_RMS),
+              "a second output joins a unit-rms update only");
+  if (y2.has_value()) {
+    check_rows(*y2);
+    y2_rs = y2->stride(0);
+  }
   if (h.has_value()) {
     check_rows(*h);
-    TORCH_CHECK(h->is_contiguous());
+    TORCH_CHECK(rows <= 1 || h->stride(0) >= W);
+    h_rs = h->stride(0);
   } else {
     TORCH_CHECK(!norm_w.has_value());
   }
@@ -314,6 +374,8 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
   const void* gp = update == UPD_GATE ? gate->data_ptr() : nullptr;
   const float* gb = gate_bias.has_value() ? gate_bias->data_ptr<float>() : nullptr;
   const float* rw = rms_w.has_value() ? rms_w->data_ptr<float>() : nullptr;
+  const void* y2p = y2.has_value() ? y2->data_ptr() : nullptr;
+  const float* rw2 = rms_w2.has_value() ? rms_w2->data_ptr<float>() : nullptr;
   const float* nw = norm_w.has_value() ? norm_w->data_ptr<float>() : nullptr;
   const float* nb = norm_b.has_value() ? norm_b->data_ptr<float>() : nullptr;
   const float* ar = add_rows.has_value() ? add_rows->data_ptr<float>() : nullptr;
@@ -324,7 +386,8 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
   hipLaunchKernelGGL((residual_update_norm_kernel<TT, V, N>), dim3(rows),     \
                      dim3(256), 0, stream, x.data_ptr<float>(),               \
                      (const TT*)yp, y_rs, (int)update, (const TT*)gp, g_rs,   \
-                     gb, rw, (float)eps, nw, nb, rms_norm, ar, av, (TT*)hp, W)
+                     gb, rw, (const TT*)y2p, y2_rs, rw2, (float)eps, nw, nb,  \
+                     rms_norm, ar, av, (TT*)hp, h_rs, W)
   const bool bf = ct == at::kBFloat16;
   TORCH_CHECK(bf || ct == at::kFloat, "expected bf16 or fp32 rows");
   if (vec) {
@@ -340,6 +403,32 @@ void residual_update_norm(torch::Tensor x, c10::optional<torch::Tensor> y,
     TORCH_CHECK(W <= 256 * 32, "unaligned row wider than 8192");
     if (bf) LAUNCH(short, 1, 32); else LAUNCH(float, 1, 32);
   }
+#undef LAUNCH
+}
+
+void relu_square(torch::Tensor out, torch::Tensor z) {
+  TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && z.dim() == 2 &&
+              z.sizes() == out.sizes() && z.stride(1) == 1 &&
+              z.scalar_type() == out.scalar_type());
+  const long n = out.numel();
+  const int C = out.size(1);
+  if (n == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+#define LAUNCH(TT, V)                                                         \
+  hipLaunchKernelGGL((relu_square_kernel<TT, V>),                             \
+                     dim3((n / V + 255) / 256), dim3(256), 0, stream,         \
+                     (TT*)out.data_ptr(), (const TT*)z.data_ptr(),            \
+                     (long)z.stride(0), n, C)
+  if (out.scalar_type() == at::kBFloat16 && C % 8 == 0 && aligned_rows(z, 8) &&
+      reinterpret_cast<uintptr_t>(out.data_ptr()) % 16 == 0 &&
+      reinterpret_cast<uintptr_t>(z.data_ptr()) % 16 == 0) {
+    LAUNCH(short, 8);
+    return;
+  }
+  const bool vec = C % 4 == 0 && aligned_rows(z, 4);
+  LATENT_DISPATCH_T(out, {
+    if (vec) LAUNCH(T, 4); else LAUNCH(T, 1);
+  });
 #undef LAUNCH
 }
 

@@ -1,7 +1,11 @@
 // Masked grouped-query attention over paged per-head K/V pools (gfx950).
 //
-//   k_cache [P, G, PS, D]   v_cache [P, G, PS, Dv]   (a page holds, per kv
+//   k_cache [P, G, PS, D]   v_cache [P, G, PS, Vs]   (a page holds, per kv
 //   head, PS consecutive token rows: one (page, head) block is contiguous)
+//   Vs = Dv; or Vs < Dv = D where values and keys agree in all coordinates
+//   from Vs on (tied values: only rotated coordinates differ): a value is
+//   its Vs pooled coordinates followed by the key row's from Vs on, which
+//   are cached once and, in a tile, still hot from the score product.
 //   q [T, H, D], out [T, H, Dv]; query head h reads kv head h / (H/G).
 //
 //   score  = <q, k> * scale;  score <- cap * tanh(score / cap)   (cap > 0)
@@ -9,7 +13,8 @@
 //   mask   : causal   j <= p
 //            window   j <= p and (p - j < size  or  j < keep)
 //            chunk    j <= p and floor(p/size) == floor(j/size)
-//   weight : softmax over the visible keys, or sigmoid(score + bias[h])
+//   weight : softmax over the visible keys (exp(sink[h]) joins the
+//            denominator when a sink is given), or sigmoid(score + bias[h])
 //            per visible key with no normalization
 //   out    = sum_j weight_j v_j  (* sigmoid(gate[t, h]) when a gate is given;
 //            a gate of heads * Dv columns gates every output coordinate:
@@ -82,6 +87,17 @@ __device__ __forceinline__ float fast_dist_penalty(float r1, float r2, int d) {
   return r1 * 0.6931471805599453f * __log2f(fmaf(r2, (float)max(d, 0), 1.0f));
 }
 
+// what a head's weighted sum with running maximum m and mass l is multiplied
+// by: 1 / l, or with a sink score s, 1 / (l + e^(s - m)) on a common maximum
+__device__ __forceinline__ float softmax_tail(float m, float l,
+                                              const float* sink, int h) {
+  if (sink == nullptr) return 1.0f / l;
+  const float s = sink[h];
+  const float mn = fmaxf(m, s);
+  const float f = expf(m - mn);
+  return f / fmaf(l, f, expf(s - mn));
+}
+
 // token position -> (page index in the sequence's table, row in the page);
 // page sizes that are powers of two (ps_shift >= 0) avoid the division
 __device__ __forceinline__ void page_of(int j, int PS, int ps_shift, int& pg,
@@ -115,8 +131,9 @@ __global__ __launch_bounds__(64) void masked_attn_rowwave_kernel(
     const int* __restrict__ q_starts, const int* __restrict__ q_lens,
     float scale, int kind, int size, int keep, int sigmoid_w, float softcap,
     const float* __restrict__ key_bias, const T* __restrict__ gate, long g_ts,
-    int gate_elem, const float* __restrict__ dist, int H, int G, int D, int Dv,
-    int PS, int max_pages, int vec) {
+    int gate_elem, const float* __restrict__ dist,
+    const float* __restrict__ sink, int H, int G, int D, int Dv, int Vs, int PS,
+    int max_pages, int vec) {
   extern __shared__ float smem[];
   float* q_s = smem;       // [D]
   float* p_s = smem + D;   // [64]
@@ -190,17 +207,19 @@ __global__ __launch_bounds__(64) void masked_attn_rowwave_kernel(
     for (int jj = 0; jj < n; ++jj) {
       const int ug = u0 + jj;
       const int jg = ug < ns ? ug : lo + (ug - ns);
-      const T* vr = vc + ((((long)pt[jg / PS] * G + g) * PS) + jg % PS) * Dv;
+      const long vrow = (((long)pt[jg / PS] * G + g) * PS) + jg % PS;
+      const T* vr = vc + vrow * Vs;
+      const T* kr = kc + vrow * D;
       const float pj = p_s[jj];
 #pragma unroll
       for (int k = 0; k < RW_MAX_ACC; ++k) {
         const int d = k * WAVE + lane;
-        if (d < Dv) acc[k] = fmaf(pj, ldf(vr, d), acc[k]);
+        if (d < Dv) acc[k] = fmaf(pj, ldf(d < Vs ? vr : kr, d), acc[k]);
       }
     }
     __syncthreads();
   }
-  float mul = sigmoid_w ? 1.0f : 1.0f / l;
+  float mul = sigmoid_w ? 1.0f : softmax_tail(m, l, sink, h);
   if (gate != nullptr && !gate_elem)
     mul *= sigmoidf_(ldf(gate, rowi * g_ts + h));
 #pragma unroll
@@ -241,8 +260,8 @@ __global__ __launch_bounds__(256) void masked_attn_mfma_kernel(
     const int* __restrict__ q_lens, float scale, int kind, int size, int keep,
     int sigmoid_w, float softcap, const float* __restrict__ key_bias,
     const short* __restrict__ gate, long g_ts, int gate_elem,
-    const float* __restrict__ dist, int H, int G, int nd, int nv, int PS,
-    int max_pages, int ps_shift) {
+    const float* __restrict__ dist, const float* __restrict__ sink, int H, int G,
+    int nd, int nv, int Vs, int PS, int max_pages, int ps_shift) {
   extern __shared__ __attribute__((aligned(16))) short lds[];
   constexpr int KL = NDB / 2;              // 16-byte K loads per thread
   const int D = nd * 32, Dv = nv * 16;
@@ -325,6 +344,8 @@ __global__ __launch_bounds__(256) void masked_attn_mfma_kernel(
   bf16x8 kreg[KL], vreg[4];
   const bool v_unit = tid < 8 * vchunks;
   const int v_kq = tid / vchunks, v_ch = tid % vchunks;
+  const short* v_src = (v_ch * 8 < Vs ? vc : kc) + v_ch * 8;
+  const int v_rs = v_ch * 8 < Vs ? Vs : D;
   auto load_tile = [&](int kt) {
     const int t0 = kt * KVT;
 #pragma unroll
@@ -350,7 +371,7 @@ __global__ __launch_bounds__(256) void masked_attn_mfma_kernel(
         int pg, off;
         page_of(j, PS, ps_shift, pg, off);
         const long row = ((long)pt[pg] * G + g) * PS + off;
-        vreg[r] = *reinterpret_cast<const bf16x8*>(vc + row * Dv + v_ch * 8);
+        vreg[r] = *reinterpret_cast<const bf16x8*>(v_src + row * v_rs);
       }
     }
   };
@@ -460,7 +481,7 @@ __global__ __launch_bounds__(256) void masked_attn_mfma_kernel(
 
   // ---- epilogue: lane holds O^T[i*16 + lg*4 + r][column]
   if (!col_ok) return;
-  float mul = sigmoid_w ? 1.0f : 1.0f / l;
+  float mul = sigmoid_w ? 1.0f : softmax_tail(m, l, sink, h);
   if (gate != nullptr && !gate_elem)
     mul *= sigmoidf_(bits2f(gate[(row_base + qi) * g_ts + h]));
   const short* ge = (gate != nullptr && gate_elem)
@@ -512,9 +533,9 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
     const int* __restrict__ seq_lens, float scale, int kind, int size, int keep,
     int sigmoid_w, float softcap, const float* __restrict__ key_bias,
     const short* __restrict__ gate, long g_ts, int gate_elem,
-    const float* __restrict__ dist, int H, int G, int nd, int nv, int PS,
-    int max_pages, int ps_shift, float* __restrict__ part_o,
-    float* __restrict__ part_ml, int n_splits) {
+    const float* __restrict__ dist, const float* __restrict__ sink, int H, int G,
+    int nd, int nv, int Vs, int PS, int max_pages, int ps_shift,
+    float* __restrict__ part_o, float* __restrict__ part_ml, int n_splits) {
   extern __shared__ __attribute__((aligned(16))) short lds[];
   const int D = nd * 32, Dv = nv * 16;
   const int split = blockIdx.x, b = blockIdx.y, g = blockIdx.z;
@@ -578,7 +599,8 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
   const int vchunks = Dv / 8;                       // = 2 * nv
   // this lane's (key quad, chunk) units of a tile's V rows
   constexpr int VU = (NVB + 3) / 4;
-  int u_kq[VU], u_ch[VU];
+  int u_kq[VU], u_ch[VU], u_rs[VU];
+  const short* u_src[VU];
   bool u_ok[VU];
 #pragma unroll
   for (int it = 0; it < VU; ++it) {
@@ -586,6 +608,8 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
     u_ok[it] = u < 8 * vchunks;
     u_kq[it] = u / vchunks;
     u_ch[it] = u % vchunks;
+    u_src[it] = (u_ch[it] * 8 < Vs ? vc : kc) + u_ch[it] * 8;
+    u_rs[it] = u_ch[it] * 8 < Vs ? Vs : D;
   }
 
   for (int v = split * 4 + wid; v < n_vt; v += 4 * n_splits) {
@@ -618,12 +642,12 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
         int pg, off;
         page_of(jq < total ? jq : 0, PS, ps_shift, pg, off);
         const short* vrow =
-            vc + (((long)pt[pg] * G + g) * PS + off) * Dv + u_ch[it] * 8;
+            u_src[it] + (((long)pt[pg] * G + g) * PS + off) * u_rs[it];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           vr[it][r] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
           if (u_ok[it] && jq + r < total)
-            vr[it][r] = *reinterpret_cast<const bf16x8*>(vrow + r * Dv);
+            vr[it][r] = *reinterpret_cast<const bf16x8*>(vrow + r * u_rs[it]);
         }
       } else {
 #pragma unroll
@@ -635,7 +659,7 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
             page_of(j, PS, ps_shift, pg, off);
             const long row = ((long)pt[pg] * G + g) * PS + off;
             vr[it][r] = *reinterpret_cast<const bf16x8*>(
-                vc + row * Dv + u_ch[it] * 8);
+                u_src[it] + row * u_rs[it]);
           }
         }
       }
@@ -750,7 +774,7 @@ __global__ __launch_bounds__(256) void masked_attn_decode_kernel(
       O = fmaf(fo[(w * Dv + e) * 16 + c], f, O);
     }
     if (n_splits == 1) {
-      float mul = sigmoid_w ? 1.0f : 1.0f / L;
+      float mul = sigmoid_w ? 1.0f : softmax_tail(M, L, sink, g * R + c);
       if (gate != nullptr)
         mul *= sigmoidf_(bits2f(
             gate[(long)b * g_ts +
@@ -771,7 +795,7 @@ __global__ __launch_bounds__(64) void masked_attn_combine_kernel(
     short* __restrict__ out, long o_ts, long o_hs,
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const short* __restrict__ gate, long g_ts, int gate_elem, int sigmoid_w,
-    int H, int G, int Dv, int n_splits) {
+    const float* __restrict__ sink, int H, int G, int Dv, int n_splits) {
   const int b = blockIdx.x, h = blockIdx.y;
   const int R = H / G, g = h / R, c = h % R;
   const long base = (long)(b * G + g) * n_splits;
@@ -784,7 +808,7 @@ __global__ __launch_bounds__(64) void masked_attn_combine_kernel(
         sigmoid_w ? 1.0f : expf(part_ml[((base + s) * R + c) * 2] - M);
     L = fmaf(part_ml[((base + s) * R + c) * 2 + 1], f, L);
   }
-  float mul = sigmoid_w ? 1.0f : (L > 0.f ? 1.0f / L : 0.f);
+  float mul = sigmoid_w ? 1.0f : (L > 0.f ? softmax_tail(M, L, sink, h) : 0.f);
   if (gate != nullptr && !gate_elem)
     mul *= sigmoidf_(bits2f(gate[(long)b * g_ts + h]));
   for (int e = threadIdx.x; e < Dv; e += WAVE) {
@@ -816,7 +840,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       c10::optional<torch::Tensor> key_bias,
                       c10::optional<torch::Tensor> head_gate, long max_qlen,
                       bool force_simple, long splits,
-                      c10::optional<torch::Tensor> dist_bias) {
+                      c10::optional<torch::Tensor> dist_bias,
+                      c10::optional<torch::Tensor> sink) {
   TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && q.stride(2) == 1 &&
               out.stride(2) == 1);
   const int T_ = q.size(0), H = q.size(1), D = q.size(2), Dv = out.size(2);
@@ -824,9 +849,13 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
   TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() &&
               v_cache.dim() == 4 && v_cache.is_contiguous());
   const int G = k_cache.size(1), PS = k_cache.size(2);
-  TORCH_CHECK(k_cache.size(3) == D && v_cache.size(3) == Dv &&
-              v_cache.size(1) == G && v_cache.size(2) == PS &&
-              v_cache.size(0) == k_cache.size(0), "pool shapes disagree");
+  const int Vs = v_cache.size(3);
+  TORCH_CHECK(k_cache.size(3) == D && v_cache.size(1) == G &&
+              v_cache.size(2) == PS && v_cache.size(0) == k_cache.size(0),
+              "pool shapes disagree");
+  TORCH_CHECK(Vs == Dv || (Dv == D && Vs >= 1 && Vs < Dv),
+              "the value pool holds whole values, or the leading coordinates "
+              "of values that end like their keys");
   TORCH_CHECK(G >= 1 && H % G == 0, "heads % kv_heads != 0");
   TORCH_CHECK(q.scalar_type() == out.scalar_type() &&
               k_cache.scalar_type() == q.scalar_type() &&
@@ -879,6 +908,13 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                 "dist_bias is fp32 [heads, 2]");
     db = dist_bias->data_ptr<float>();
   }
+  const float* sk = nullptr;
+  if (sink.has_value()) {
+    TORCH_CHECK(sink->scalar_type() == at::kFloat && sink->numel() == H &&
+                sink->is_contiguous(), "sink is fp32 [heads]");
+    TORCH_CHECK(!sigmoid_weights, "a sink needs softmax weights");
+    sk = sink->data_ptr<float>();
+  }
   if (T_ == 0 || B == 0) return;
   const int keep = mask_kind == MK_WINDOW ? (int)keep_first : 0;
   auto stream = at::hip::getCurrentHIPStream();
@@ -886,7 +922,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
 
   const bool mfma_ok =
       q.scalar_type() == at::kBFloat16 && !force_simple && D % 32 == 0 &&
-      D <= 256 && Dv % 16 == 0 && Dv <= 256 && q.stride(0) % 8 == 0 &&
+      D <= 256 && Dv % 16 == 0 && Dv <= 256 && Vs % 8 == 0 &&
+      q.stride(0) % 8 == 0 &&
       q.stride(1) % 8 == 0 && out.stride(0) % 4 == 0 && out.stride(1) % 4 == 0 &&
       aligned16(q.data_ptr()) && aligned16(out.data_ptr()) &&
       aligned16(k_cache.data_ptr()) && aligned16(v_cache.data_ptr());
@@ -927,8 +964,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                      page_table.data_ptr<int>(), seq_lens.data_ptr<int>(),    \
                      (float)scale, (int)mask_kind, (int)mask_size, keep,      \
                      sigmoid_weights ? 1 : 0, (float)softcap, kb, gp, g_ts,   \
-                     gate_elem, db, H, G, nd, nv, PS, max_pages, ps_shift,    \
-                     pop, pmlp, (int)n_splits)
+                     gate_elem, db, sk, H, G, nd, nv, Vs, PS, max_pages,      \
+                     ps_shift, pop, pmlp, (int)n_splits)
       if (nd <= 4 && nv <= 4) {
         LAUNCH_DECODE(4, 4);
       } else if (nd <= 4 && nv <= 8) {
@@ -941,7 +978,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
         hipLaunchKernelGGL(masked_attn_combine_kernel, dim3(B, H), dim3(64), 0,
                            stream, (short*)out.data_ptr(), (long)out.stride(0),
                            (long)out.stride(1), pop, pmlp, gp, g_ts, gate_elem,
-                           sigmoid_weights ? 1 : 0, H, G, Dv, (int)n_splits);
+                           sigmoid_weights ? 1 : 0, sk, H, G, Dv,
+                           (int)n_splits);
       }
       return;
     }
@@ -958,7 +996,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                      page_table.data_ptr<int>(), seq_lens.data_ptr<int>(), qs, \
                      ql, (float)scale, (int)mask_kind, (int)mask_size, keep,  \
                      sigmoid_weights ? 1 : 0, (float)softcap, kb, gp, g_ts,   \
-                     gate_elem, db, H, G, nd, nv, PS, max_pages, ps_shift)
+                     gate_elem, db, sk, H, G, nd, nv, Vs, PS, max_pages,      \
+                     ps_shift)
     if (nd <= 4 && nv <= 4) {
       LAUNCH_MFMA(4, 4);
     } else if (nd <= 4 && nv <= 8) {
@@ -985,7 +1024,7 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
         (const T*)k_cache.data_ptr(), (const T*)v_cache.data_ptr(),
         page_table.data_ptr<int>(), seq_lens.data_ptr<int>(), qs, ql,
         (float)scale, (int)mask_kind, (int)mask_size, keep,
-        sigmoid_weights ? 1 : 0, (float)softcap, kb, gp, g_ts, gate_elem, db, H,
-        G, D, Dv, PS, max_pages, vec);
+        sigmoid_weights ? 1 : 0, (float)softcap, kb, gp, g_ts, gate_elem, db, sk,
+        H, G, D, Dv, Vs, PS, max_pages, vec);
   });
 }

@@ -1,5 +1,5 @@
 // pybind11 bindings: scalar-gain norms, PolyNorm, rotary + q/k norm + K/V
-// append, masked grouped-query attention.
+// append, row-wide q/k norm + K/V append, masked grouped-query attention.
 #include <torch/extension.h>
 
 void scalar_postnorm_residual(torch::Tensor x, torch::Tensor y,
@@ -14,7 +14,12 @@ void rotary_norm_append(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                         torch::Tensor k_cache, torch::Tensor v_cache,
                         torch::Tensor cos_sin, torch::Tensor slot_mapping,
                         double eps, c10::optional<torch::Tensor> q_w,
-                        c10::optional<torch::Tensor> k_w, bool norm_first);
+                        c10::optional<torch::Tensor> k_w, long norm);
+void row_norm_append(torch::Tensor q, torch::Tensor k, torch::Tensor v,
+                     torch::Tensor k_cache, torch::Tensor v_cache,
+                     torch::Tensor positions, torch::Tensor slot_mapping,
+                     double eps, torch::Tensor q_w, torch::Tensor k_w,
+                     double temp_coef, long temp_every);
 void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       torch::Tensor v_cache, torch::Tensor page_table,
                       torch::Tensor seq_lens,
@@ -25,7 +30,8 @@ void masked_attention(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
                       c10::optional<torch::Tensor> key_bias,
                       c10::optional<torch::Tensor> head_gate, long max_qlen,
                       bool force_simple, long splits,
-                      c10::optional<torch::Tensor> dist_bias);
+                      c10::optional<torch::Tensor> dist_bias,
+                      c10::optional<torch::Tensor> sink);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "agentainer_amd CDNA4 (gfx950) masked-attention family kernels";
@@ -36,8 +42,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rotary_table", &rotary_table,
         "cos | sin of position * frequency for one step's tokens");
   m.def("rotary_norm_append", &rotary_norm_append,
-        "rotary + q/k rms norm; append K/V to the paged pools");
+        "rotary (+ q/k rms norm); append K/V to the paged pools");
+  m.def("row_norm_append", &row_norm_append,
+        "q/k rms norm over all heads, query temperature; append K/V");
   m.def("masked_attention", &masked_attention,
-        "chunk / window masked GQA with softmax or sigmoid weights and an "
-        "optional logarithmic distance bias");
+        "chunk / window masked GQA with softmax (optional sink) or sigmoid "
+        "weights and an optional logarithmic distance bias");
 }

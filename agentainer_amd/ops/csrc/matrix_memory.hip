@@ -1,18 +1,20 @@
 // Matrix-memory recurrences over per-sequence state (gfx950): gated linear
 // attention, gated delta rule with per-key-channel decay or with one decay
-// per head, and the mLSTM
-// memory with a running-maximum stabilizer — plus the per-head output norm
-// and gate that follow them.
+// per head, the mLSTM memory with a running-maximum stabilizer, and the
+// state-space (Mamba-2) recurrence — plus the output norms and gates that
+// follow them.
 //
 // Per head the memory S has `D` key rows and `Dv` value columns; every
 // column evolves on its own given the token's k, q and decays:
 //
-//   S'   = g (.) S                      (g: per key row; mLSTM and the
-//                                        head-decay delta rule: one number)
+//   S'   = g (.) S                      (g: per key row; mLSTM, the head-
+//                                        decay delta rule and the state-
+//                                        space recurrence: one number)
 //   a1_j = sum_r S'[r, j] k[r]          (delta rules only)
 //   a2_j = sum_r S'[r, j] q[r]
-//   u_j  = beta (v_j - a1_j)  |  v_j  |  e^(i - m') v_j
+//   u_j  = beta (v_j - a1_j)  |  v_j  |  e^(i - m') v_j  |  step v_j
 //   S    = S' + k u^T,   o_j = a2_j + u_j (k . q)     [= (S^T q)_j]
+//                              (+ skip_h v_j in the state-space recurrence)
 //
 // so the work is cut over (sequence, head, block of value columns): a wave
 // owns 64 / NSUB columns, NSUB adjacent lanes share a column and split its
@@ -46,6 +48,7 @@ void launch_delta(const ScanArgs& a, int B, int lanes, bool bf16,
                   hipStream_t s);
 void launch_delta_head(const ScanArgs& a, int B, int lanes, bool bf16,
                        hipStream_t s);
+void launch_ssd(const ScanArgs& a, int B, int lanes, bool bf16, hipStream_t s);
 void launch_mlstm(const ScanArgs& a, int B, int lanes, bool bf16,
                   hipStream_t s);
 }  // namespace mm
@@ -56,6 +59,7 @@ using mm::KIND_GLA;
 using mm::KIND_DELTA;
 using mm::KIND_DELTA_HEAD;
 using mm::KIND_MLSTM;
+using mm::KIND_SSD;
 using mm::ScanArgs;
 
 // Per-key-channel decays, evaluated once per token and channel by a fully
@@ -168,7 +172,107 @@ __global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(
   st4(out, row * Dv + i, v);
 }
 
+// ---- gate first, then RMS norm over equal parts of the row ---------------
+//   out = (o silu(z)) / sqrt(mean over the part of its square + eps) * w
+// TPR threads (a wave or the workgroup) own one part of one row and keep its
+// gated values in registers (NREG groups of VEC).
+template <typename T, int TPR, int VEC, int NREG>
+__global__ __launch_bounds__(256) void gate_group_norm_kernel(
+    T* __restrict__ out, const float* __restrict__ o,
+    const float* __restrict__ w, const T* __restrict__ z, long z_rs, float eps,
+    long n_rows, int parts, int L) {
+  __shared__ float red[4];
+  const long row = (long)blockIdx.x * (256 / TPR) + threadIdx.x / TPR;  // (t, part)
+  if (row >= n_rows) return;           // whole waves; TPR = 256: never taken
+  const int lane = threadIdx.x % TPR;
+  const long t = row / parts;
+  const int c0 = (int)(row - t * parts) * L;
+  float v[NREG][VEC];
+  float ss = 0.f;
+#pragma unroll
+  for (int r = 0; r < NREG; ++r) {
+    const int i = (r * TPR + lane) * VEC;
+    if (i < L) {
+      float g[VEC];
+      if constexpr (VEC == 4) {
+        ld4(o, row * L + i, v[r]);
+        ld4(z, t * z_rs + c0 + i, g);
+      } else {
+        v[r][0] = o[row * L + i];
+        g[0] = ldf(z, t * z_rs + c0 + i);
+      }
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        v[r][e] *= g[e] / (1.0f + expf(-g[e]));
+        ss = fmaf(v[r][e], v[r][e], ss);
+      }
+    }
+  }
+  if constexpr (TPR == 64) ss = wave_sum(ss); else ss = block_sum_256(ss, red);
+  const float m = 1.0f / sqrtf(ss / (float)L + eps);
+#pragma unroll
+  for (int r = 0; r < NREG; ++r) {
+    const int i = (r * TPR + lane) * VEC;
+    if (i < L) {
+      if constexpr (VEC == 4) {
+        float wv[4];
+        ld4(w, c0 + i, wv);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[r][e] *= m * wv[e];
+        st4(out, row * L + i, v[r]);
+      } else {
+        stf(out, row * L + i, v[r][0] * m * w[c0 + i]);
+      }
+    }
+  }
+}
+
 }  // namespace
+
+void gate_group_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor w,
+                        torch::Tensor z, long parts, double eps) {
+  TORCH_CHECK(o.scalar_type() == at::kFloat && o.is_contiguous() &&
+              o.dim() == 2);
+  const int T_ = o.size(0), C = o.size(1);
+  TORCH_CHECK(parts >= 1 && C % parts == 0, "unequal norm parts");
+  const int L = C / parts;
+  TORCH_CHECK(out.is_contiguous() && out.sizes() == o.sizes());
+  TORCH_CHECK(w.scalar_type() == at::kFloat && w.is_contiguous() &&
+              w.numel() == C);
+  TORCH_CHECK(z.sizes() == o.sizes() && z.stride(1) == 1 &&
+              z.scalar_type() == out.scalar_type());
+  const long n_rows = (long)T_ * parts;
+  if (n_rows == 0) return;
+  TORCH_CHECK(L <= 8192, "norm part wider than 8192");
+  auto stream = at::hip::getCurrentHIPStream();
+  const bool vec = L % 4 == 0 && z.stride(0) % 4 == 0 &&
+                   reinterpret_cast<uintptr_t>(z.data_ptr()) %
+                           (4 * z.element_size()) == 0;
+#define LAUNCH(TPR, V, N)                                                     \
+  hipLaunchKernelGGL((gate_group_norm_kernel<T, TPR, V, N>),                  \
+                     dim3((n_rows + 256 / TPR - 1) / (256 / TPR)), dim3(256), \
+                     0, stream, (T*)out.data_ptr(), o.data_ptr<float>(),      \
+                     w.data_ptr<float>(), (const T*)z.data_ptr(),             \
+                     (long)z.stride(0), (float)eps, n_rows, (int)parts, L)
+  LATENT_DISPATCH_T(out, {
+    if (!vec) {
+      if (L <= 512) LAUNCH(64, 1, 8); else LAUNCH(256, 1, 32);
+    } else if (L <= 256) {
+      LAUNCH(64, 4, 1);
+    } else if (L <= 512) {
+      LAUNCH(64, 4, 2);
+    } else if (L <= 1024) {
+      LAUNCH(256, 4, 1);
+    } else if (L <= 2048) {
+      LAUNCH(256, 4, 2);
+    } else if (L <= 4096) {
+      LAUNCH(256, 4, 4);
+    } else {
+      LAUNCH(256, 4, 8);
+    }
+  });
+#undef LAUNCH
+}
 
 void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
                         torch::Tensor k, torch::Tensor v, torch::Tensor gate,
@@ -180,8 +284,9 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
                         c10::optional<torch::Tensor> m_state,
                         torch::Tensor state_slots, torch::Tensor seq_lens,
                         c10::optional<torch::Tensor> query_starts,
-                        c10::optional<torch::Tensor> query_lens, long lanes) {
-  TORCH_CHECK(kind >= 0 && kind <= 3, "unknown recurrence");
+                        c10::optional<torch::Tensor> query_lens, long lanes,
+                        c10::optional<torch::Tensor> skip) {
+  TORCH_CHECK(kind >= 0 && kind <= 4, "unknown recurrence");
   TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 && out.dim() == 3);
   const int T_ = v.size(0), H = v.size(1), Dv = v.size(2);
   const int G = k.size(1), D = k.size(2);
@@ -216,19 +321,27 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
     TORCH_CHECK(G == H);
     a.n_state = n_state->data_ptr<float>();
     a.m_state = m_state->data_ptr<float>();
-  } else if (kind == KIND_DELTA_HEAD) {
+  } else if (mm::head_decay(kind)) {
     TORCH_CHECK(gate.size(1) == H && gate_bias->numel() == H);
   } else {
     TORCH_CHECK(gate.size(1) == (long)H * D && gate_bias->numel() == (long)H * D);
   }
-  if (mm::is_delta(kind)) {
-    TORCH_CHECK(head_rate.has_value() && beta.has_value());
-    TORCH_CHECK(head_rate->scalar_type() == at::kFloat &&
+  if (mm::is_delta(kind) || kind == KIND_SSD) {
+    TORCH_CHECK(head_rate.has_value() &&
+                head_rate->scalar_type() == at::kFloat &&
                 head_rate->is_contiguous() && head_rate->numel() == H);
+    a.head_rate = head_rate->data_ptr<float>();
+  }
+  if (kind == KIND_SSD) {
+    TORCH_CHECK(skip.has_value() && skip->scalar_type() == at::kFloat &&
+                skip->is_contiguous() && skip->numel() == H);
+    a.skip = skip->data_ptr<float>();
+  }
+  if (mm::is_delta(kind)) {
+    TORCH_CHECK(beta.has_value());
     TORCH_CHECK(beta->scalar_type() == at::kFloat && beta->dim() == 2 &&
                 beta->size(0) == T_ && beta->size(1) == H &&
                 beta->stride(1) == 1);
-    a.head_rate = head_rate->data_ptr<float>();
     a.beta = beta->data_ptr<float>();
     a.beta_rs = beta->stride(0);
   }
@@ -294,6 +407,7 @@ void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
   else if (kind == KIND_DELTA) mm::launch_delta(a, B, (int)lanes, bf16, stream);
   else if (kind == KIND_DELTA_HEAD)
     mm::launch_delta_head(a, B, (int)lanes, bf16, stream);
+  else if (kind == KIND_SSD) mm::launch_ssd(a, B, (int)lanes, bf16, stream);
   else mm::launch_mlstm(a, B, (int)lanes, bf16, stream);
   if (kind == KIND_MLSTM) {
     hipLaunchKernelGGL(scatter_nm_kernel, dim3((H * D + 255) / 256, B),

@@ -8,7 +8,8 @@
 
 namespace mm {
 
-constexpr int KIND_GLA = 0, KIND_DELTA = 1, KIND_MLSTM = 2, KIND_DELTA_HEAD = 3;
+constexpr int KIND_GLA = 0, KIND_DELTA = 1, KIND_MLSTM = 2, KIND_DELTA_HEAD = 3,
+              KIND_SSD = 4;
 // delta rules correct the memory towards v; the other kinds add k v^T
 constexpr bool is_delta(int kind) {
   return kind == KIND_DELTA || kind == KIND_DELTA_HEAD;
@@ -16,6 +17,11 @@ constexpr bool is_delta(int kind) {
 // decays per key channel (staged vectors) or one number per head and token
 constexpr bool channel_decay(int kind) {
   return kind == KIND_GLA || kind == KIND_DELTA;
+}
+// decay (and write scale) evaluated inside the kernel, one number per head
+// and token
+constexpr bool head_decay(int kind) {
+  return kind == KIND_DELTA_HEAD || kind == KIND_SSD;
 }
 constexpr int CH = 8;      // tokens staged together
 constexpr int WAVES = 4;   // waves of a workgroup; they share the staging
@@ -28,9 +34,11 @@ struct ScanArgs {
   const void* v;         // [T, H, Dv]
   const float* gate;     // gla / delta: decays [T, H*D], already evaluated;
                          // mLSTM: gate pre-activations [T, 2H];
-                         // head delta: decay pre-activations [T, H]
+                         // head delta, ssd: decay / step-size
+                         // pre-activations [T, H]
   const float* gate_bias;
-  const float* head_rate;  // [H] (head delta)
+  const float* head_rate;  // [H] (head delta, ssd)
+  const float* skip;       // [H] (ssd)
   const float* beta;     // [T, H], row stride beta_rs
   float* S;              // [slots, H, Dv, D]
   const float* n_state;  // [slots, H, D]   (read at the start)
@@ -89,7 +97,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
   __shared__ __attribute__((aligned(16))) float kbuf[CH][ROWS];
   __shared__ __attribute__((aligned(16))) float qbuf[CH][ROWS];
   __shared__ __attribute__((aligned(16))) float gbuf[channel_decay(KIND) ? CH : 1][ROWS];
-  __shared__ float sc[CH][4];   // k.q | write scale (beta, e^(i-m)) | one-number decay | e^(-m')
+  __shared__ float sc[CH][4];   // k.q | write scale (beta, e^(i-m), step) | one-number decay | e^(-m')
 
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int col = lane / NSUB, sub = lane % NSUB;
@@ -141,7 +149,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
   // ---- raw inputs of the next chunk, in registers. Wave w stages the
   // tokens c = w, w + WAVES, ... of a chunk for the whole workgroup; every
   // lane keeps its own column's v; wave 0 evaluates the mLSTM gates, the
-  // last wave the head-decay rule's two numbers, lane c those of token c.
+  // last wave the head-decay rules' two numbers, lane c those of token c.
   float rk[TPW][EPL], rq[TPW][EPL], rg[channel_decay(KIND) ? TPW : 1][EPL];
   float rb[TPW];
   float rv[CH];
@@ -180,21 +188,23 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         rgf = a.gate[row * a.gate_rs + H + h];
       }
     }
-    if constexpr (KIND == KIND_DELTA_HEAD) {
+    if constexpr (head_decay(KIND)) {
       if (wave == WAVES - 1 && lane < CH && t0 + lane < n_tok) {
         const long row = s0 + t0 + lane;
         rgi = a.gate[row * a.gate_rs + h];
-        rgf = a.beta[row * a.beta_rs + h];
+        if constexpr (KIND == KIND_DELTA_HEAD)
+          rgf = a.beta[row * a.beta_rs + h];
       }
     }
   };
 
   float bias_i = 0.f, bias_f = 0.f;
-  float rate = 0.f;
-  if constexpr (KIND == KIND_DELTA_HEAD) {
+  float rate = 0.f, skip = 0.f;
+  if constexpr (head_decay(KIND)) {
     bias_i = a.gate_bias[h];
     rate = expf(a.head_rate[h]);
   }
+  if constexpr (KIND == KIND_SSD) skip = a.skip[h];
   if constexpr (KIND == KIND_MLSTM) {
     bias_i = a.gate_bias[h];
     bias_f = a.gate_bias[H + h];
@@ -229,10 +239,11 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         }
       }
     }
-    if constexpr (KIND == KIND_DELTA_HEAD) {
+    if constexpr (head_decay(KIND)) {
       if (wave == WAVES - 1 && lane < CH && t0 + lane < n_tok) {
-        sc[lane][1] = 1.0f / (1.0f + expf(-rgf));
-        sc[lane][2] = expf(-rate * soft_plus(rgi + bias_i));
+        const float step = soft_plus(rgi + bias_i);
+        sc[lane][1] = KIND == KIND_SSD ? step : 1.0f / (1.0f + expf(-rgf));
+        sc[lane][2] = expf(-rate * step);
       }
     }
     if constexpr (KIND == KIND_MLSTM) {
@@ -309,7 +320,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
         if constexpr (is_delta(KIND)) {
           const float a1s = sub_sum<NSUB>((a1[0] + a1[1]) + (a1[2] + a1[3]));
           u = cu[c] * (cv[c] - a1s);
-        } else if constexpr (KIND == KIND_MLSTM) {
+        } else if constexpr (KIND == KIND_MLSTM || KIND == KIND_SSD) {
           u = cu[c] * cv[c];
         } else {
           u = cv[c];
@@ -324,6 +335,7 @@ __global__ __launch_bounds__(256) void scan_kernel(const ScanArgs a) {
           S[i4 * 4 + 3] = fmaf(k4.w, u, S[i4 * 4 + 3]);
         }
         float o = fmaf(u, ckq[c], a2s);
+        if constexpr (KIND == KIND_SSD) o = fmaf(skip, cv[c], o);
         if constexpr (KIND == KIND_MLSTM) {
           const float nqs = sub_sum<NSUB>((nq[0] + nq[1]) + (nq[2] + nq[3]));
           o = o / (fmaxf(fabsf(nqs), cei[c]) + 1e-6f);
@@ -380,7 +392,7 @@ void launch_scan(const ScanArgs& a, int B, int lanes, hipStream_t stream) {
     ns = lanes < lo ? lo : (lanes > 16 ? 16 : lanes);
   } else {
     const long cols = (long)B * a.H * a.Dv;
-    if constexpr (KIND == KIND_DELTA_HEAD) {
+    if constexpr (head_decay(KIND)) {
       // with no decay vectors to read, 16 rows per lane beat both 8 and 32
       // from about a thousand waves on
       ns = lo * 2 < 16 ? lo * 2 : 16;

@@ -13,16 +13,18 @@ void short_conv_state(torch::Tensor out, torch::Tensor u, torch::Tensor w,
                       torch::Tensor seq_lens, OptT query_starts,
                       OptT query_lens, bool silu, long norm_channels,
                       long head_dim, long lead_channels, double lead_scale,
-                      double l2_eps);
+                      double l2_eps, OptT bias);
 void matrix_memory_scan(long kind, torch::Tensor out, torch::Tensor q,
                         torch::Tensor k, torch::Tensor v, torch::Tensor gate,
                         OptT gate_bias, OptT head_rate, OptT beta,
                         double q_scale, double gate_param, torch::Tensor S,
                         OptT n_state, OptT m_state, torch::Tensor state_slots,
                         torch::Tensor seq_lens, OptT query_starts,
-                        OptT query_lens, long lanes);
+                        OptT query_lens, long lanes, OptT skip);
 void head_rmsnorm_gate(torch::Tensor out, torch::Tensor o, torch::Tensor w,
                        torch::Tensor gate, double eps, bool silu_gate);
+void gate_group_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor w,
+                        torch::Tensor z, long parts, double eps);
 void grouped_softmax_route(torch::Tensor weight, torch::Tensor logits,
                            OptT correction, long top, long n_groups,
                            long keep_groups, double scale);
@@ -36,9 +38,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("short_conv_state", &short_conv_state,
         "depthwise causal convolution with a per-sequence tail");
   m.def("matrix_memory_scan", &matrix_memory_scan,
-        "gated linear attention / gated delta rules / mLSTM over state");
+        "gated linear attention / gated delta rules / mLSTM / state-space "
+        "recurrence over state");
   m.def("head_rmsnorm_gate", &head_rmsnorm_gate,
         "per-head RMS norm, weight and output gate");
+  m.def("gate_group_rmsnorm", &gate_group_rmsnorm,
+        "o * silu(z), RMS-normed in equal parts, times weight");
   m.def("grouped_softmax_route", &grouped_softmax_route,
         "softmax scores, group-limited top-k, renormalized weights");
   m.def("routed_clamped_glu", &routed_clamped_glu,

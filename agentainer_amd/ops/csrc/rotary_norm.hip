@@ -7,8 +7,9 @@
 //                        every layer and head with that setting reads it.
 //   rotary_norm_append   for every new token and head, in fp32:
 //
-//     norm_first : u <- u / sqrt(mean(u^2) + eps) * w ;  u <- rotate(u)
-//     otherwise  : u <- rotate(u) ;  u <- u / sqrt(mean(u^2) + eps)
+//     norm first : u <- u / sqrt(mean(u^2) + eps) * w ;  u <- rotate(u)
+//     norm last  : u <- rotate(u) ;  u <- u / sqrt(mean(u^2) + eps)
+//     no norm    : u <- rotate(u)
 //
 // rotate() turns the first 2*half coordinates of the head, coordinate i
 // paired with i + half; coordinates from 2*half on pass through. `amp` is 1
@@ -30,6 +31,7 @@
 
 namespace {
 
+constexpr int NORM_LAST = 0, NORM_FIRST = 1, NORM_OFF = 2;
 constexpr int RN_WAVES = 4;
 constexpr int RN_PAIRS = 2;   // rotation pairs per lane: rotary dims <= 256
 constexpr int RN_PASS = 4;    // pass-through values per lane: <= 256
@@ -53,7 +55,7 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_kernel(
     T* __restrict__ k_cache, T* __restrict__ v_cache,
     const float* __restrict__ cos_sin, int half,
     const long* __restrict__ slots, float eps, const float* __restrict__ q_w,
-    const float* __restrict__ k_w, int norm_first, int n_tok, int H, int G,
+    const float* __restrict__ k_w, int norm, int n_tok, int H, int G,
     int D, int Dv, int PS) {
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int per_tok = H + 2 * G;
@@ -79,11 +81,11 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_kernel(
                         : k + (long)t * k_ts + (long)(j - H) * k_hs;
     const float* w = is_q ? q_w : k_w;
     // every load of the head is issued before the first use: head values,
-    // the token's cos/sin and (norm_first) the norm weights
+    // the token's cos/sin and (norm first) the norm weights
     float a[RN_PAIRS], b[RN_PAIRS], c[RN_PASS];
     float cc[RN_PAIRS], sn[RN_PAIRS];
     float wa[RN_PAIRS], wb[RN_PAIRS], wc[RN_PASS];
-    const bool use_w = norm_first && w != nullptr;
+    const bool use_w = norm == NORM_FIRST && w != nullptr;
 #pragma unroll
     for (int n = 0; n < RN_PAIRS; ++n) {
       const int i = lane + n * WAVE;
@@ -102,7 +104,7 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_kernel(
       wc[n] = (i < D && use_w) ? w[i] : 1.f;
     }
     float ss = 0.f;
-    if (norm_first) {
+    if (norm == NORM_FIRST) {
 #pragma unroll
       for (int n = 0; n < RN_PAIRS; ++n)
         ss = fmaf(a[n], a[n], fmaf(b[n], b[n], ss));
@@ -126,7 +128,7 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_kernel(
       ss = fmaf(a[n], a[n], fmaf(b[n], b[n], ss));
     }
     float r = 1.0f;
-    if (!norm_first) {
+    if (norm == NORM_LAST) {
 #pragma unroll
       for (int n = 0; n < RN_PASS; ++n) ss = fmaf(c[n], c[n], ss);
       r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
@@ -210,7 +212,7 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_vec_kernel(
     short* __restrict__ k_cache, short* __restrict__ v_cache,
     const float* __restrict__ cos_sin, int half,
     const long* __restrict__ slots, float eps, const float* __restrict__ q_w,
-    const float* __restrict__ k_w, int norm_first, int n_tok, int H, int G,
+    const float* __restrict__ k_w, int norm, int n_tok, int H, int G,
     int Dv, int PS) {
   constexpr int D = WAVE * EPL;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
@@ -246,8 +248,8 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_vec_kernel(
     ld_f<EPL>(cs + i0, cc);
     ld_f<EPL>(cs + half + i0, sn);
   }
-  if (norm_first && w != nullptr) ld_f<EPL>(w + e0, wv);
-  if (norm_first) {
+  if (norm == NORM_FIRST && w != nullptr) ld_f<EPL>(w + e0, wv);
+  if (norm == NORM_FIRST) {
     float ss = 0.f;
 #pragma unroll
     for (int e = 0; e < EPL; ++e) ss = fmaf(x[e], x[e], ss);
@@ -266,7 +268,7 @@ __global__ __launch_bounds__(64 * RN_WAVES) void rotary_norm_append_vec_kernel(
     x[e] = turns ? rx : x[e];
     ss = fmaf(x[e], x[e], ss);
   }
-  if (!norm_first) {
+  if (norm == NORM_LAST) {
     const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
 #pragma unroll
     for (int e = 0; e < EPL; ++e) x[e] *= r;
@@ -303,7 +305,8 @@ void rotary_norm_append(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                         torch::Tensor k_cache, torch::Tensor v_cache,
                         torch::Tensor cos_sin, torch::Tensor slot_mapping,
                         double eps, c10::optional<torch::Tensor> q_w,
-                        c10::optional<torch::Tensor> k_w, bool norm_first) {
+                        c10::optional<torch::Tensor> k_w, long norm) {
+  TORCH_CHECK(norm >= NORM_LAST && norm <= NORM_OFF);
   TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.dim() == 3 &&
               q.stride(2) == 1 && k.stride(2) == 1 && v.stride(2) == 1);
   const int T_ = q.size(0), H = q.size(1), D = q.size(2);
@@ -369,7 +372,7 @@ void rotary_norm_append(torch::Tensor q, torch::Tensor k, torch::Tensor v,
       (const short*)v.data_ptr(), (long)v.stride(0), (long)v.stride(1),       \
       (short*)k_cache.data_ptr(), (short*)v_cache.data_ptr(),                 \
       cos_sin.data_ptr<float>(), half, slot_mapping.data_ptr<long>(),         \
-      (float)eps, qw, kw, norm_first ? 1 : 0, T_, H, G, Dv,                   \
+      (float)eps, qw, kw, (int)norm, T_, H, G, Dv,                   \
       (int)k_cache.size(2))
     if (epl == 1) {
       LAUNCH_VEC(1);
@@ -390,7 +393,7 @@ void rotary_norm_append(torch::Tensor q, torch::Tensor k, torch::Tensor v,
         (long)k.stride(1), (const T*)v.data_ptr(), (long)v.stride(0),
         (long)v.stride(1), (T*)k_cache.data_ptr(), (T*)v_cache.data_ptr(),
         cos_sin.data_ptr<float>(), half, slot_mapping.data_ptr<long>(),
-        (float)eps, qw, kw, norm_first ? 1 : 0, T_, H, G, D, Dv,
+        (float)eps, qw, kw, (int)norm, T_, H, G, D, Dv,
         (int)k_cache.size(2));
   });
 }

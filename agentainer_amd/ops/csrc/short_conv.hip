@@ -1,7 +1,7 @@
 // Depthwise short causal convolution over time with a per-sequence tail
 // (gfx950).
 //
-//   y[t, c] = sum_j w[j, c] * u[t - taps + 1 + j, c]      (w is [taps, C])
+//   y[t, c] = bias[c] + sum_j w[j, c] * u[t - taps + 1 + j, c]   (w [taps, C])
 //
 // over a step's token rows (variable-length portions of several sequences,
 // or one new token per sequence). Inputs before the step's first row come
@@ -26,7 +26,7 @@
 
 namespace {
 
-constexpr int MAX_TAPS = 8;
+constexpr int MAX_TAPS = 64;   // sanity bound, nothing is sized by it
 constexpr int MAXV = 8;   // channels per lane: chunks of up to 512 channels
 
 // sequence of token row t: the last b with starts[b] <= t
@@ -42,7 +42,8 @@ __device__ __forceinline__ int find_seq(const int* starts, int B, int t) {
 template <typename TI, typename TO>
 __global__ __launch_bounds__(256) void short_conv_kernel(
     TO* __restrict__ out, long out_rs, const TI* __restrict__ u, long u_rs,
-    const float* __restrict__ w, const float* __restrict__ tail,
+    const float* __restrict__ w, const float* __restrict__ bias,
+    const float* __restrict__ tail,
     const long* __restrict__ slots, const int* __restrict__ seq_lens,
     const int* __restrict__ q_starts, const int* __restrict__ q_lens, int B,
     int C, int taps, int cs, int n_chunks, int nyb, bool silu,
@@ -73,7 +74,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
     const int c = c0 + e * 64 + lane;
     yv[e] = 0.f;
     if (e * 64 + lane < cs && c < C) {
-      float acc = 0.f;
+      float acc = bias ? bias[c] : 0.f;
       for (int j = 0; j < taps; ++j) {
         const int src = off - (taps - 1) + j;   // row within the portion
         float uv = 0.f;
@@ -109,7 +110,8 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
 template <typename TI, typename TO, int LPH>
 __global__ __launch_bounds__(256) void short_conv_vec_kernel(
     TO* __restrict__ out, long out_rs, const TI* __restrict__ u, long u_rs,
-    const float* __restrict__ w, const float* __restrict__ tail,
+    const float* __restrict__ w, const float* __restrict__ bias,
+    const float* __restrict__ tail,
     const long* __restrict__ slots, const int* __restrict__ seq_lens,
     const int* __restrict__ q_starts, const int* __restrict__ q_lens, int B,
     int C, int taps, int cs, int n_chunks, int nyb, bool silu,
@@ -135,6 +137,7 @@ __global__ __launch_bounds__(256) void short_conv_vec_kernel(
   const bool active = chunk < n_chunks && li * 4 < cs && c < C;
   float acc[4] = {0.f, 0.f, 0.f, 0.f};
   if (active) {
+    if (bias) ld4(bias, c, acc);
     for (int j = 0; j < taps; ++j) {
       const int src = off - (taps - 1) + j;
       float uv[4] = {0.f, 0.f, 0.f, 0.f};
@@ -206,7 +209,8 @@ void short_conv_state(torch::Tensor out, torch::Tensor u, torch::Tensor w,
                       c10::optional<torch::Tensor> query_starts,
                       c10::optional<torch::Tensor> query_lens, bool silu,
                       long norm_channels, long head_dim, long lead_channels,
-                      double lead_scale, double l2_eps) {
+                      double lead_scale, double l2_eps,
+                      c10::optional<torch::Tensor> bias) {
   TORCH_CHECK(u.dim() == 2 && u.stride(1) == 1 && out.dim() == 2 &&
               out.stride(1) == 1);
   const int T_ = u.size(0), C = u.size(1);
@@ -215,6 +219,12 @@ void short_conv_state(torch::Tensor out, torch::Tensor u, torch::Tensor w,
               w.dim() == 2 && w.size(1) == C, "weights must be [taps, C]");
   const int taps = w.size(0);
   TORCH_CHECK(taps >= 1 && taps <= MAX_TAPS, "unsupported tap count");
+  const float* bp = nullptr;
+  if (bias.has_value()) {
+    TORCH_CHECK(bias->scalar_type() == at::kFloat && bias->is_contiguous() &&
+                bias->numel() == C, "bias must be fp32 [C]");
+    bp = bias->data_ptr<float>();
+  }
   TORCH_CHECK(tail.scalar_type() == at::kFloat && tail.is_contiguous() &&
               tail.dim() == 3 && tail.size(1) == taps - 1 && tail.size(2) == C,
               "tail must be fp32 [slots, taps-1, channels]");
@@ -256,14 +266,15 @@ void short_conv_state(torch::Tensor out, torch::Tensor u, torch::Tensor w,
                      dim3(256), 0, stream,                                    \
                      (TO*)out.data_ptr(), (long)out.stride(0),                \
                      (const TI*)u.data_ptr(), (long)u.stride(0),              \
-                     w.data_ptr<float>(), tail.data_ptr<float>(),             \
+                     w.data_ptr<float>(), bp, tail.data_ptr<float>(),         \
                      state_slots.data_ptr<long>(), seq_lens.data_ptr<int>(),  \
                      qs, ql, B, C, taps, cs, n_chunks, (n_chunks + 3) / 4,    \
                      silu, (int)norm_channels, (int)lead_channels,            \
                      (float)lead_scale, (float)l2_eps)
   const bool vec = cs % 4 == 0 && cs <= 256 && C % 4 == 0 &&
                    u.stride(0) % 4 == 0 && out.stride(0) % 4 == 0 &&
-                   u.storage_offset() % 4 == 0 && out.storage_offset() % 4 == 0;
+                   u.storage_offset() % 4 == 0 && out.storage_offset() % 4 == 0 &&
+                   (bp == nullptr || reinterpret_cast<uintptr_t>(bp) % 16 == 0);
   int lph = 1;
   while (lph * 4 < cs) lph <<= 1;
 #define LAUNCH_VEC(TI, TO, L)                                                 \
@@ -272,7 +283,7 @@ void short_conv_state(torch::Tensor out, torch::Tensor u, torch::Tensor w,
                                                  (4 * (64 / L))))),           \
                      dim3(256), 0, stream, (TO*)out.data_ptr(),               \
                      (long)out.stride(0), (const TI*)u.data_ptr(),            \
-                     (long)u.stride(0), w.data_ptr<float>(),                  \
+                     (long)u.stride(0), w.data_ptr<float>(), bp,              \
                      tail.data_ptr<float>(), state_slots.data_ptr<long>(),    \
                      seq_lens.data_ptr<int>(), qs, ql, B, C, taps, cs,        \
                      n_chunks, (n_chunks + 4 * (64 / L) - 1) / (4 * (64 / L)), \

@@ -413,22 +413,28 @@ def _rotate_half(u: torch.Tensor, cos_sin: torch.Tensor) -> torch.Tensor:
     return torch.cat([a * c - b * s, b * c + a * s, u[..., 2 * half:]], -1)
 
 
+NORM_LAST, NORM_FIRST, NORM_OFF = 0, 1, 2
+
+
 def rotary_norm_append(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
                        k_cache: torch.Tensor, v_cache: torch.Tensor,
                        cos_sin: torch.Tensor, slot_mapping: torch.Tensor,
                        eps: float, q_w=None, k_w=None,
-                       norm_first: bool = False) -> None:
+                       norm: int = NORM_LAST) -> None:
     """Prepare one step's queries and keys and append K/V to the pools.
 
     q [T, H, D] (rewritten in place), k [T, G, D], v [T, G, Dv]; pools
     k_cache [P, G, PS, D], v_cache [P, G, PS, Dv] (per page and kv head, PS
     consecutive token rows); slot = page*PS + offset (slot < 0 skips the
     append); cos_sin = rotary_table(...) of the step. Per head, in fp32:
-      norm_first: u <- rms_norm(u) * w, then rotate   (w = q_w / k_w [D])
-      otherwise : u <- rotate(u), then unit rms (no weight)."""
+      NORM_FIRST: u <- rms_norm(u) * w, then rotate   (w = q_w / k_w [D])
+      NORM_LAST : u <- rotate(u), then unit rms (no weight)
+      NORM_OFF  : u <- rotate(u)."""
     def prep(u, w):
         u = u.float()
-        if norm_first:
+        if norm == NORM_OFF:
+            return _rotate_half(u, cos_sin)
+        if norm == NORM_FIRST:
             u = _unit(u, eps)
             if w is not None:
                 u = u * w.float()
@@ -443,6 +449,26 @@ def rotary_norm_append(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
     page, off = rows // PS, rows % PS
     k_cache[page, :, off] = kk[ok]
     v_cache[page, :, off] = v[ok].to(v_cache.dtype)
+
+
+def row_norm_append(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
+                    k_cache: torch.Tensor, v_cache: torch.Tensor,
+                    positions: torch.Tensor, slot_mapping: torch.Tensor,
+                    eps: float, q_w: torch.Tensor, k_w: torch.Tensor,
+                    temp_coef: float, temp_every: int) -> None:
+    """Weighted RMS norm over ALL heads of a token at once: q [T, H*D] is
+    rewritten in place and multiplied by 1 + temp_coef * ln(floor((p + 1) /
+    temp_every) + 1) at position p; k [T, G*D] goes normed into k_cache
+    [P, G, PS, D], v [T, G*Dv] as it is into v_cache (slot < 0 skips)."""
+    temp = 1.0 + temp_coef * torch.log(
+        (torch.div(positions.long() + 1, temp_every, rounding_mode="floor")
+         + 1).float())
+    q.copy_((_unit(q.float(), eps) * q_w.float() * temp.unsqueeze(1)
+             ).to(q.dtype))
+    kk = (_unit(k.float(), eps) * k_w.float()).to(k_cache.dtype)
+    T, G = k.size(0), k_cache.size(1)
+    head_kv_append(kk.view(T, G, -1), v.reshape(T, G, -1), k_cache, v_cache,
+                   slot_mapping)
 
 
 MASK_CAUSAL, MASK_WINDOW, MASK_CHUNK = 0, 1, 2
@@ -468,7 +494,7 @@ def masked_attention(out: torch.Tensor, q: torch.Tensor,
                      query_starts, query_lens, scale: float, mask_kind: int,
                      mask_size: int, keep_first: int, sigmoid_weights: bool,
                      softcap: float, key_bias, head_gate,
-                     dist_bias=None) -> None:
+                     dist_bias=None, sink=None) -> None:
     """Grouped-query attention over paged per-head K/V pools.
 
     out [T, H, Dv], q [T, H, D]; query head h reads kv head h // (H/G).
@@ -480,7 +506,11 @@ def masked_attention(out: torch.Tensor, q: torch.Tensor,
     output coordinate. query_starts/query_lens None means
     one new token per sequence; rows with seq_len <= 0 come back zero.
     dist_bias fp32 [H, 2] = (r1, r2) per head takes r1 * ln(1 + r2 * (p - j))
-    off the (capped) score of key j for the query at position p."""
+    off the (capped) score of key j for the query at position p. sink fp32
+    [H]: exp(sink_h) joins head h's softmax denominator, with no key and no
+    value. When v_cache's rows are shorter than Dv they hold a value's leading
+    coordinates and the key row's coordinates from there on complete it
+    (D == Dv)."""
     H = q.size(1)
     G, PS = k_cache.size(1), k_cache.size(2)
     rep = H // G
@@ -497,6 +527,8 @@ def masked_attention(out: torch.Tensor, q: torch.Tensor,
         pages = page_table[b, (pos // PS).long()].long()
         K = k_cache[pages, :, pos % PS].float().repeat_interleave(rep, dim=1)
         V = v_cache[pages, :, pos % PS].float().repeat_interleave(rep, dim=1)
+        if V.size(2) < out.size(2):
+            V = torch.cat([V, K[..., V.size(2):]], dim=-1)
         Q = q[start:start + qlen].float()                     # K [n, H, D]
         s = torch.einsum("qhd,nhd->hqn", Q, K) * scale
         if softcap > 0:
@@ -514,7 +546,11 @@ def masked_attention(out: torch.Tensor, q: torch.Tensor,
                 s = s + key_bias.float().view(H, 1, 1)
             p = torch.sigmoid(s) * seen
         else:
-            p = torch.softmax(s.masked_fill(~seen, float("-inf")), dim=-1)
+            s = s.masked_fill(~seen, float("-inf"))
+            if sink is not None:
+                s = torch.cat([s, sink.float().view(H, 1, 1).expand(
+                    H, qlen, 1)], dim=-1)
+            p = torch.softmax(s, dim=-1)[..., :total]
         o = torch.einsum("hqn,nhe->qhe", p, V)
         if head_gate is not None:
             gt = torch.sigmoid(head_gate[start:start + qlen].float())
@@ -566,12 +602,12 @@ def short_conv_state(out: torch.Tensor, u: torch.Tensor, w: torch.Tensor,
                      tail: torch.Tensor, state_slots: torch.Tensor,
                      seq_lens, query_starts, query_lens, silu: bool,
                      norm_channels: int, head_dim: int, lead_channels: int,
-                     lead_scale: float, l2_eps: float) -> None:
+                     lead_scale: float, l2_eps: float, bias=None) -> None:
     """Depthwise causal convolution over time with the last taps-1 inputs
     of every sequence kept in tail [slots, taps-1, C] (fp32).
 
-    y[t, c] = sum_j w[j, c] * u[t - taps + 1 + j, c] (w is tap-major,
-    [taps, C]); inputs before this
+    y[t, c] = bias[c] + sum_j w[j, c] * u[t - taps + 1 + j, c] (w is
+    tap-major, [taps, C]; bias None: 0); inputs before this
     step's rows come from the tail, inputs before position 0 are zero (a
     sequence whose first row sits at position 0 ignores its tail). Then
     optionally silu, and for the first norm_channels channels, cut into
@@ -588,6 +624,8 @@ def short_conv_state(out: torch.Tensor, u: torch.Tensor, w: torch.Tensor,
         hist[:max(0, taps - 1 - max(pos0, 0))] = 0      # before position 0
         full = torch.cat([hist, u[s0:s0 + n].float()], dim=0)
         y = torch.zeros(n, u.size(1))
+        if bias is not None:
+            y = y + bias.float()
         for j in range(taps):
             y = y + wf[j] * full[j:j + n]
         if taps > 1:
@@ -602,7 +640,7 @@ def short_conv_state(out: torch.Tensor, u: torch.Tensor, w: torch.Tensor,
         out[s0:s0 + n] = y.to(out.dtype)
 
 
-SCAN_GLA, SCAN_DELTA, SCAN_MLSTM, SCAN_DELTA_HEAD = 0, 1, 2, 3
+SCAN_GLA, SCAN_DELTA, SCAN_MLSTM, SCAN_DELTA_HEAD, SCAN_SSD = 0, 1, 2, 3, 4
 
 
 def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
@@ -610,7 +648,7 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
                        gate_bias, head_rate, beta, q_scale: float,
                        gate_param: float, S: torch.Tensor, n_state, m_state,
                        state_slots: torch.Tensor, seq_lens, query_starts,
-                       query_lens) -> None:
+                       query_lens, skip=None) -> None:
     """Token-by-token matrix-memory recurrences over per-sequence state.
 
     q, k [T, G, D]; v [T, H, Dv]; out [T, H, Dv] fp32; head h reads q/k
@@ -624,6 +662,9 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
                 b = sigmoid(beta[t, h]); S <- g S; u = b (v - S^T k);
                 S <- S + k u^T; o = S^T q. gate [T, H*D].
     SCAN_DELTA_HEAD: the same rule with one decay per head (gate [T, H]).
+    SCAN_SSD:   step = softplus(gate + gate_bias) per head (gate [T, H]);
+                S <- exp(-exp(head_rate[h]) * step) S + step * k v^T;
+                o = S^T q + skip[h] * v.
     SCAN_MLSTM: gate [T, 2H] = log-input | forget pre-activations,
                 i = c tanh((gate_i + bias_i) / c), f = logsigmoid(c tanh(
                 (gate_f + bias_f) / c)), c = gate_param; m' = max(f + m, i);
@@ -663,6 +704,13 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
                 u = bt * (vt - torch.einsum("hvd,hd->hv", St, kt))
                 St = St + u.unsqueeze(2) * kt.unsqueeze(1)
                 out[t] = torch.einsum("hvd,hd->hv", St, qt)
+            elif kind == SCAN_SSD:
+                step = torch.nn.functional.softplus(z + gb)
+                g = torch.exp(-torch.exp(head_rate.float()) * step)
+                St = (St * g.view(H, 1, 1) + (step.view(H, 1) * vt
+                                              ).unsqueeze(2) * kt.unsqueeze(1))
+                out[t] = (torch.einsum("hvd,hd->hv", St, qt)
+                          + skip.float().view(H, 1) * vt)
             else:
                 c = gate_param
                 zb = z + gb
@@ -682,6 +730,16 @@ def matrix_memory_scan(kind: int, out: torch.Tensor, q: torch.Tensor,
         if kind == SCAN_MLSTM:
             n_state[slot] = nv
             m_state[slot] = mv
+
+
+def gate_group_rmsnorm(out: torch.Tensor, o: torch.Tensor, w: torch.Tensor,
+                       z: torch.Tensor, parts: int, eps: float) -> None:
+    """out = (o * silu(z)), every one of `parts` equal consecutive parts of a
+    row divided by its own root mean square, times w [C]. o fp32 [T, C]."""
+    zf = z.float()
+    g = o * (zf * torch.sigmoid(zf))
+    g = _unit(g.view(g.size(0), parts, -1), eps).reshape(o.shape)
+    out.copy_((g * w.float()).to(out.dtype))
 
 
 def head_rmsnorm_gate(out: torch.Tensor, o: torch.Tensor, w: torch.Tensor,
@@ -752,7 +810,16 @@ def routed_clamped_glu(out: torch.Tensor, gu: torch.Tensor,
 # rotary append, plain K/V append, elementwise output gate.
 # ---------------------------------------------------------------------
 
-UPDATE_NONE, UPDATE_SIGMOID_GATE, UPDATE_UNIT_RMS = 0, 1, 2
+UPDATE_NONE, UPDATE_SIGMOID_GATE, UPDATE_UNIT_RMS, UPDATE_ADD = 0, 1, 2, 3
+
+
+def embed_rows(ids: torch.Tensor, embed: torch.Tensor, x_out, raw) -> None:
+    """x_out (fp32) and / or raw (the table's type) = embed[ids]."""
+    rows = embed[ids]
+    if x_out is not None:
+        x_out.copy_(rows.float())
+    if raw is not None:
+        raw.copy_(rows)
 
 
 def bigram_embed(x_out: torch.Tensor, ids: torch.Tensor, embed: torch.Tensor,
@@ -787,10 +854,11 @@ def bigram_embed(x_out: torch.Tensor, ids: torch.Tensor, embed: torch.Tensor,
 def residual_update_norm(x_res: torch.Tensor, y, update: int, gate, gate_bias,
                          rms_w, eps: float, norm_w, norm_b, h_out,
                          rms_norm: bool = False, add_rows=None,
-                         add_vec=None) -> None:
+                         add_vec=None, y2=None, rms_w2=None) -> None:
     """fp32 residual update fused with the norm that feeds the next GEMM.
     update: NONE; SIGMOID_GATE x += sigmoid(gate + gate_bias) * y;
-    UNIT_RMS x += y / sqrt(mean(y^2) + eps) * rms_w. Then x += add_rows +
+    UNIT_RMS x += y / sqrt(mean(y^2) + eps) * rms_w (and the same of y2,
+    rms_w2 when given); ADD x += y. Then x += add_rows +
     add_vec where given. Then h_out = layer
     norm of x ((x - mean) / sqrt(var + eps) * norm_w + norm_b; rms_norm:
     x / sqrt(mean(x^2) + eps) * norm_w + norm_b), or just x
@@ -802,6 +870,10 @@ def residual_update_norm(x_res: torch.Tensor, y, update: int, gate, gate_bias,
         x_res.add_(torch.sigmoid(g) * y.float())
     elif update == UPDATE_UNIT_RMS:
         x_res.add_(_unit(y.float(), eps) * rms_w.float())
+        if y2 is not None:
+            x_res.add_(_unit(y2.float(), eps) * rms_w2.float())
+    elif update == UPDATE_ADD:
+        x_res.add_(y.float())
     if add_rows is not None:
         x_res.add_(add_rows)
     if add_vec is not None:
@@ -830,6 +902,10 @@ def position_embed_norm(x_out: torch.Tensor, ids: torch.Tensor,
     x_out.copy_(_unit(v, eps) * w.float())
     if x_copy is not None:
         x_copy.copy_(x_out)
+
+
+def relu_square(out: torch.Tensor, z: torch.Tensor) -> None:
+    out.copy_(z.float().clamp(min=0.0).pow(2).to(out.dtype))
 
 
 def xielu(out: torch.Tensor, z: torch.Tensor, coef: torch.Tensor) -> None:
