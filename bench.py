@@ -87,7 +87,7 @@ def _parser():
                         "(default: all points of the design)")
     p.add_argument("--arch-design", default="lelitar",
                    choices=["lelitar", "volalorn", "pekarax", "sipelorn",
-                            "mugazen"],
+                            "mugazen", "larozen"],
                    help="--arch-compare: which design to measure")
     return p
 
@@ -347,11 +347,59 @@ def _mugazen_points():
     }
 
 
+def _larozen_points():
+    """Larozen size points: four layer runs (a tied-value attention layer
+    that runs twice, rotary on half the head, then two parallel layers:
+    positionless attention beside a state-space recurrence with an inner
+    size of twice the width, heads of 64 channels x 128 states in 8 groups),
+    every one followed by the squared-ReLU feed-forward. 's' and 'l' stand
+    beside the Volalorn stacks of equal width, attention heads and ff (the
+    closest existing family: masked attention, two-matrix dense
+    feed-forward), 's-llama' and 'l-llama' beside Llama, 's-pek' beside the
+    Pekarax stack (attention beside a matrix memory)."""
+    from agentainer_amd import ops
+    from agentainer_amd.models.larozen import (LarozenConfig,
+                                               LarozenLayerConfig,
+                                               StateSpaceConfig)
+    from agentainer_amd.models.volalorn import MaskedAttentionConfig
+
+    def lar(name, width, heads, kv, ff):
+        common = dict(heads=heads, kv_heads=kv, dim=128, vdim=128,
+                      scale=128 ** -0.5, mask_kind=ops.MASK_CAUSAL,
+                      mask_size=0, qkv_bias=True)
+        tied = MaskedAttentionConfig(
+            rot_dims=64, rot_base=500000.0, rot_pairs=True, rotate_only=True,
+            tied_values=True, softcap=50.0, **common)
+        left = MaskedAttentionConfig(
+            row_norm=True, sink=True, out_bias=True, q_temp_coef=0.1,
+            q_temp_every=8192, **common)
+        right = StateSpaceConfig(heads=2 * width // 64, vdim=64, state=128,
+                                 groups=8, conv_taps=4, norm_groups=8)
+        layers = [LarozenLayerConfig("attention", tied, ff=ff),
+                  LarozenLayerConfig("parallel", left, right, ff=ff),
+                  LarozenLayerConfig("parallel", left, right, ff=ff)]
+        return LarozenConfig(name=name, vocab_size=32000, hidden_size=width,
+                             layers=layers, norm_eps=1e-5, loop_start=0,
+                             loop_stop=1, loop_times=2)
+
+    s = lar("larozen-s", 2048, 16, 4, 8192)
+    lg = lar("larozen-l", 4096, 32, 8, 14336)
+    vol = _volalorn_points()
+    return {
+        "s": ("w2048-ff8192", s, vol["s"][1], "volalorn"),
+        "l": ("w4096-ff14336", lg, vol["l"][1], "volalorn"),
+        "s-llama": ("w2048-ff8192", s, vol["s"][2], None),
+        "l-llama": ("w4096-ff14336", lg, vol["l"][2], None),
+        "s-pek": ("w2048-ff8192", s, _pekarax_points()["s"][1], "pekarax"),
+    }
+
+
 def run_arch_compare(args):
     """Prefill (8 x 1024-token prompts per step) and decode (64 sequences at
     1024 tokens of context, captured graph) throughput, through the
     engine's own varlen and decode step functions."""
     from agentainer_amd.engine.llm import ModelInstance
+    from agentainer_amd.models.larozen import LarozenForCausalLM
     from agentainer_amd.models.lelitar import LelitarForCausalLM
     from agentainer_amd.models.mixtral import MixtralForCausalLM
     from agentainer_amd.models.mugazen import MugazenForCausalLM
@@ -418,13 +466,16 @@ def run_arch_compare(args):
     design = args.arch_design
     pts = {"volalorn": _volalorn_points, "pekarax": _pekarax_points,
            "sipelorn": _sipelorn_points, "mugazen": _mugazen_points,
+           "larozen": _larozen_points,
            "lelitar": _arch_points}[design]()
     cls_of = {"mixtral": MixtralForCausalLM, "pekarax": PekaraxForCausalLM,
-              "sipelorn": SipelornForCausalLM}
+              "sipelorn": SipelornForCausalLM,
+              "volalorn": VolalornForCausalLM}
     ours_cls = {"volalorn": VolalornForCausalLM,
                 "pekarax": PekaraxForCausalLM,
                 "sipelorn": SipelornForCausalLM,
                 "mugazen": MugazenForCausalLM,
+                "larozen": LarozenForCausalLM,
                 "lelitar": LelitarForCausalLM}[design]
     for key in (args.arch_sizes or ",".join(pts)).split(","):
         label, lcfg, rcfg, kind = pts[key.strip()]

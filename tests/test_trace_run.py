@@ -12,6 +12,7 @@ import torch
 
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
+import larozen_oracle as LO  # noqa: E402
 import lelitar_oracle as O  # noqa: E402
 import mugazen_oracle as MO  # noqa: E402
 import pekarax_oracle as PO  # noqa: E402
@@ -82,9 +83,26 @@ def _mugazen_case():
     return _MugazenOracle, cfg, MO.random_weights(cfg, seed=25)
 
 
+class _LarozenOracle:
+    """The Larozen oracle behind the other oracles' call signature."""
+    save_checkpoint = staticmethod(LO.save_checkpoint)
+
+    @staticmethod
+    def forward(cfg, w, tokens):
+        return LO.forward(tokens, w, cfg).float()
+
+
+def _larozen_case():
+    cfg = LO.make_config(
+        [(LO.attention_layer(), 40), (LO.parallel_layer(), 30),
+         (LO.attention_layer(dim=8, rot_dims=8), None)], vocab=120,
+        loop=(0, 2, 2))
+    return _LarozenOracle, cfg, LO.random_weights(cfg, seed=26)
+
+
 @pytest.mark.parametrize("case", [_lelitar_case, _volalorn_case,
                                   _pekarax_case, _sipelorn_case,
-                                  _mugazen_case])
+                                  _mugazen_case, _larozen_case])
 def test_trace_run_mixed_steps_match_oracle(tmp_path, case):
     O, cfg, w = case()
     model = str(tmp_path / "ckpt")
