@@ -124,7 +124,9 @@ def test_sandwich_residual_with_pass_inputs(device, dtype, W):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("T,N,K", [(1, 1, 64), (3, 8, 40), (70, 33, 256),
                                    (17, 130, 72), (2100, 64, 512),
-                                   (2100, 20, 96), (5, 6, 50), (33, 16, 4096)])
+                                   (2100, 20, 96), (5, 6, 50), (33, 16, 4096),
+                                   (8200, 70, 96), (8200, 60, 264),
+                                   (4100, 150, 520)])
 def test_narrow_projection_keeps_32_bits(device, dtype, T, N, K):
     wide = rnd(T, K + 8, seed=1)
     x = wide[:, 8:]                      # a view with an offset
